@@ -107,6 +107,12 @@ class EngineConfig:
     def stage_size(self) -> int:
         return self.dp_size * self.tp_size
 
+    def cap_model_length(self, rows: int) -> None:
+        """Clamp ``model_max_length`` to what the model can place: a
+        learned position table has ``rows`` rows (0: no such limit)."""
+        if rows:
+            self.model_max_length = min(self.model_max_length or rows, rows)
+
     def torch_dtype(self):
         import torch
         return {

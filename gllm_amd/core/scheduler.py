@@ -106,7 +106,19 @@ class Scheduler:
     # intake / abort
     # ------------------------------------------------------------------
     def add_seqs(self, seqs: List[Sequence]) -> None:
+        cap = self.config.model_max_length
         for seq in seqs:
+            if cap:
+                # no position past the model's context is ever scheduled
+                # (the last token of a full context is sampled, not run)
+                if seq.prompt_len > cap:
+                    raise ValueError(
+                        f"prompt of {seq.prompt_len} tokens exceeds the "
+                        f"model's {cap} positions")
+                room = max(1, cap - seq.prompt_len)
+                if seq.sampling.max_tokens > room:
+                    seq.sampling = dataclasses.replace(seq.sampling,
+                                                       max_tokens=room)
             self.seqs_to_prefill.append(seq)
 
     def abort_seqs(self, seq_ids) -> None:
@@ -405,6 +417,11 @@ class Scheduler:
                 raise ValueError(
                     f"seq {seq.seq_id}: cannot advance {n} tokens from "
                     f"{start} (holds {len(seq.token_ids)})")
+            cap = self.config.model_max_length
+            if cap and start + n > cap:
+                raise ValueError(
+                    f"seq {seq.seq_id}: position {start + n - 1} is past "
+                    f"the model's {cap} positions")
             pages_total = -(-(start + n) // self.page_size)
             need = max(0, pages_total - len(seq.page_table))
             plan.append((seq, start, n, need))

@@ -61,6 +61,7 @@ class AsyncLLMEngine:
         # base_port kept for CLI compat; the queue transport ignores it
         self.config = config
         self.hf_config = load_hf_config(config.model)
+        config.cap_model_length(getattr(self.hf_config, "max_positions", 0))
         self.tokenizer = self._load_tokenizer(config.model)
         eos = getattr(self.hf_config, "eos_token_id", None)
         if self.tokenizer is not None and self.tokenizer.eos_token_id is not None:
@@ -254,6 +255,14 @@ class AsyncLLMEngine:
                               self.tokenizer, loop)
             self.requests[seq_id] = st
             self.request_counter += 1
+            cap = self.config.model_max_length
+            if cap and len(token_ids) > cap:
+                # more tokens than the model has positions: refused here,
+                # the workers never see it
+                logger.warning("request of %d tokens refused: the model "
+                               "has %d positions", len(token_ids), cap)
+                self._handle_token(st, -1, "abort")
+                return st
             self.comm.send_to_all("req", {
                 "seq_id": seq_id,
                 "token_ids": token_ids,

@@ -18,6 +18,13 @@ class ReLU2(nn.Module):
         return ops.relu2(x)
 
 
+class GELU(nn.Module):
+    """Exact (erf) gelu."""
+
+    def forward(self, x):
+        return ops.gelu_erf(x)
+
+
 class XIELU(nn.Module):
     """xIELU with two learned numbers (p, q) per layer:
 

@@ -274,8 +274,8 @@ class TalkingHeadsAttention(nn.Module):
 
 
 class LatentAttention(nn.Module):
-    """Causal attention whose keys and values are up-projections of one
-    cached low-rank latent per token, without positions.
+    """Attention whose keys and values are up-projections of one cached
+    low-rank latent per token.
 
         c_t   = RMSnorm(W_dkv h_t)                  (the only cached row)
         k_j,h = W_uk,h c_j      v_j,h = W_uv,h c_j
@@ -286,21 +286,30 @@ class LatentAttention(nn.Module):
     attention runs over the latent rows themselves as one shared
     key/value head, and the per-head weighted latent is brought to the
     value space afterwards (W_uv,h applied to the sum). The cache of the
-    layer is ``[pages, page, 1, rank]`` and serves as key and value
-    cache at once.
+    layer is ``[pages, page, 1, rank + rot_dim]``; its first ``rank``
+    columns serve as key and value at once.
 
-    ``owns_kv`` False: the layer has no W_dkv and attends over the
-    latent another layer cached (``layer_idx`` names that cache), with
-    up-projections of its own.
+    * ``rot_dim`` > 0 (with ``rotary``, a PairRotary over all of it): the
+      query heads carry ``rot_dim`` more dimensions and every token one
+      more key part of that size, shared by the heads; both are turned by
+      their positions and their product joins the score
+    * ``window`` > 0: position i sees 0 <= i - j < window
+    * ``sink``: exp(sinks[h]) joins the softmax denominator (fp32 [H])
+    * ``owns_kv`` False: the layer has no W_dkv and attends over the
+      latent another layer cached (``layer_idx`` names that cache), with
+      up-projections of its own (without rotated part)
 
-    ``w_uk`` [H, D, rank] and ``w_uv`` [H, Dv, rank] are parameters of
-    this module; the down projections and their norms live in the
-    caller's merged projection.
+    ``w_uk`` [H, D, rank] and ``w_uv`` [H, rank, Dv] are parameters of
+    this module (``load_up`` takes them as stored, head by head); the
+    down projections and their norms live in the caller's merged
+    projection.
     """
 
     def __init__(self, layer_idx: int, num_heads: int, head_dim: int,
                  v_head_dim: int, rank: int, scale: float, eps: float,
-                 owns_kv: bool = True, params_dtype=None):
+                 owns_kv: bool = True, params_dtype=None, rot_dim: int = 0,
+                 rotary: Optional[nn.Module] = None, window: int = 0,
+                 sink: bool = False):
         super().__init__()
         dtype = params_dtype or torch.get_default_dtype()
         self.layer_idx = layer_idx
@@ -311,37 +320,65 @@ class LatentAttention(nn.Module):
         self.scale = scale
         self.eps = eps
         self.owns_kv = owns_kv
+        self.rot_dim = rot_dim
+        self.rotary = rotary
+        self.window = window
+        assert owns_kv or not rot_dim
+        assert not rot_dim or rotary.rot_dims == rot_dim
         self.w_uk = nn.Parameter(
             torch.empty(num_heads, head_dim, rank, dtype=dtype),
             requires_grad=False)
+        # right operand of a batched product: kept the way it is read
         self.w_uv = nn.Parameter(
-            torch.empty(num_heads, v_head_dim, rank, dtype=dtype),
+            torch.empty(num_heads, rank, v_head_dim, dtype=dtype),
             requires_grad=False)
         if owns_kv:
             self.kv_norm = nn.Parameter(torch.ones(rank, dtype=dtype),
                                         requires_grad=False)
+        if sink:
+            self.sinks = nn.Parameter(
+                torch.zeros(num_heads, dtype=torch.float32),
+                requires_grad=False)
+        else:
+            self.sinks = None
+
+    def load_up(self, which: str, w: torch.Tensor) -> None:
+        """``which`` "uk": [H*D, rank]; "uv": [H*Dv, rank]."""
+        w = w.view(self.num_heads, -1, self.rank)
+        dst = self.w_uk if which == "uk" else self.w_uv
+        if which == "uv":
+            w = w.transpose(1, 2)
+        assert w.shape == dst.shape, (tuple(w.shape), tuple(dst.shape))
+        dst.data.copy_(w.to(dst.dtype))
 
     def forward(self, q: torch.Tensor, ckv: Optional[torch.Tensor],
-                fctx: ForwardContext) -> torch.Tensor:
-        """q [T, H*D]; ckv [T, rank] = W_dkv h before its norm (None for
-        a layer that reads another layer's latent). Returns [T, H*Dv]."""
+                fctx: ForwardContext,
+                gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """q [T, H*(D + rot_dim)], head by head (its rotated part is
+        turned in place); ckv [T, rank + rot_dim] = W_dkv h before its
+        norm (None for a layer that reads another layer's latent); gate
+        [T, H*Dv] logits: every output element is multiplied by
+        sigmoid(gate). Returns [T, H*Dv]."""
         T = q.shape[0]
         H, D, Dv, R = self.num_heads, self.head_dim, self.v_head_dim, \
             self.rank
         if fctx.is_profile_run:
             return q.new_zeros(T, H * Dv)
         cache = fctx.k_caches[self.layer_idx]
-        if self.owns_kv:
+        if self.rot_dim:
+            ops.latent_rope_store(
+                q, ckv, self.kv_norm, self.eps, fctx.positions,
+                fctx.slot_mapping, self.rotary.freqs, self.rotary.mag,
+                cache, H, D, R, self.rot_dim)
+        elif self.owns_kv:
             ops.rms_weight_store(ckv, self.kv_norm, self.eps, cache,
                                  fctx.slot_mapping)
-        # q~[t, h] = W_uk,h^T q[t, h]
-        q_lat = torch.bmm(q.reshape(T, H, D).transpose(0, 1), self.w_uk)
-        q_lat = q_lat.transpose(0, 1).reshape(T, H * R)
-        o_lat = ops.window_attention(
-            q_lat, None, cache, cache, fctx.block_table, fctx.seq_lens,
-            fctx.query_start_loc, self.scale, 0, 0, False,
+        heads = q.view(T, H, D + self.rot_dim)
+        # q~[h, t] = W_uk,h^T q[t, h]
+        q_lat = torch.bmm(heads[..., :D].transpose(0, 1), self.w_uk)
+        o_lat = ops.latent_attention(
+            q_lat, heads[..., D:], cache, fctx.block_table, fctx.seq_lens,
+            fctx.query_start_loc, self.scale, self.window, self.sinks,
             fctx.max_query_len)
-        # o[t, h] = W_uv,h o~[t, h]
-        o = torch.bmm(o_lat.reshape(T, H, R).transpose(0, 1),
-                      self.w_uv.transpose(1, 2))
-        return o.transpose(0, 1).reshape(T, H * Dv)
+        # o[h, t] = W_uv,h o~[h, t]
+        return ops.head_gate(torch.bmm(o_lat, self.w_uv), gate)

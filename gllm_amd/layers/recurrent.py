@@ -180,3 +180,69 @@ class GeneralDeltaRule(nn.Module):
             fctx.query_start_loc, fctx.max_query_len)
         return ops.rms_gate(o, gate, self.norm_weight, self.heads, self.eps,
                             r.dtype, gate="sigmoid", scale=scale, out=out)
+
+
+class ChannelDeltaRule(nn.Module):
+    """Gated delta rule with a decay per (value head, key channel):
+
+        g_t = exp(-exp(A_log_h) softplus(a_logit_t + dt_bias))
+        S_t = diag(g_t) S_(t-1) + k_t (beta_t (v_t - (diag(g_t) S_(t-1))^T k_t))^T
+        o_t = S_t^T q_t,   beta_t = sigmoid(b_logit_t)
+
+    on unit queries (times ``dim ** -0.5``) and unit keys per head, with
+    ``heads`` value heads sharing ``kv_heads`` q/k heads, and a read-out
+    o / rms(o) * norm_weight * sigmoid(gate) per head (one weight row
+    [vdim] for all heads). q, k and v (one merged buffer, q | k | v) pass
+    a short causal convolution with silu first; its last taps - 1 inputs
+    live in the state pool beside the fp32 state [slots, heads, dim,
+    vdim]. The caller owns every projection; decay, write strength, unit
+    norms and the state are fp32.
+    """
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int,
+                 taps: int, eps: float, ssm_layer_id: int,
+                 params_dtype=None):
+        super().__init__()
+        assert heads % kv_heads == 0
+        dtype = params_dtype or torch.get_default_dtype()
+        self.heads, self.kv_heads = heads, kv_heads
+        self.dim, self.vdim, self.taps = dim, vdim, taps
+        self.eps = eps
+        self.ssm_layer_id = ssm_layer_id
+        self.qkv_sizes = [kv_heads * dim, kv_heads * dim, heads * vdim]
+        self.conv_dim = sum(self.qkv_sizes)
+
+        def param(*shape, fill=0.0, dtype=dtype):
+            return nn.Parameter(torch.full(shape, fill, dtype=dtype),
+                                requires_grad=False)
+
+        self.conv_weight = param(self.conv_dim, taps)
+        self.A_log = param(heads, dtype=torch.float32)
+        self.dt_bias = param(heads * dim, dtype=torch.float32)
+        self.norm_weight = param(vdim, fill=1.0)
+
+    def spec(self) -> SSMLayerSpec:
+        return SSMLayerSpec(self.conv_dim, self.taps, self.heads, self.dim,
+                            self.vdim, layout="kv")
+
+    def forward(self, qkv: torch.Tensor, a_logit: torch.Tensor,
+                b_logit: torch.Tensor, gate: torch.Tensor,
+                fctx: ForwardContext) -> torch.Tensor:
+        """qkv [T, 2*kv_heads*dim + heads*vdim] before the convolution,
+        a_logit [T, heads*dim], b_logit [T, heads], gate [T, heads*vdim]
+        (row views are fine) -> [T, heads*vdim]."""
+        T = qkv.shape[0]
+        if fctx.is_profile_run or fctx.ssm_pool is None:
+            return qkv.new_zeros(T, self.heads * self.vdim)
+        pool, sid = fctx.ssm_pool, self.ssm_layer_id
+        slots, init = state_rows(fctx, T, qkv.device)
+        qkv = ops.causal_conv_silu(
+            qkv, self.conv_weight, pool.conv_state[sid], slots, init,
+            fctx.query_start_loc, max_query_len=fctx.max_query_len)
+        q, k, v = qkv.split(self.qkv_sizes, dim=-1)
+        o = ops.channel_delta_rule(
+            q, k, v, a_logit, b_logit, self.A_log, self.dt_bias,
+            pool.ssm_state[sid], slots, init, fctx.query_start_loc,
+            self.dim ** -0.5, fctx.max_query_len)
+        return ops.rms_gate(o, gate, self.norm_weight, self.heads, self.eps,
+                            qkv.dtype, gate="sigmoid")

@@ -455,9 +455,9 @@ class GopetarForCausalLM(nn.Module):
         elif sub == ["uq"]:
             self._copy(mix.uq.weight, w)
         elif sub == ["uk"]:
-            self._copy(at.w_uk.data.view(-1, at.rank), w)
+            at.load_up("uk", w)
         elif sub == ["uv"]:
-            self._copy(at.w_uv.data.view(-1, at.rank), w)
+            at.load_up("uv", w)
         elif sub == ["o"]:
             self._copy(mix.out_proj.weight, w)
         else:

@@ -37,7 +37,9 @@ def get_arch_registry():
     from gllm_amd.models.gukirax import GukiraxForCausalLM
     from gllm_amd.models.gopetar import GopetarForCausalLM
     from gllm_amd.models.sofunex import SofunexForCausalLM
+    from gllm_amd.models.kaketar import KaketarForCausalLM
     return {
+        "Kaketar": KaketarForCausalLM,
         "Sofunex": SofunexForCausalLM,
         "Gopetar": GopetarForCausalLM,
         "Sudevik": SudevikForCausalLM,

@@ -793,23 +793,47 @@ def residual_layernorm(x: torch.Tensor, y: torch.Tensor, w_post, b_post,
 
 def stream_rmsnorm(x: torch.Tensor, y, w_post, eps: float,
                    mult: float = 1.0, y_scale: float = 1.0, y2=None,
-                   add=None, pre_w=None):
-    """One launch per sublayer boundary of an RMS sandwich-norm decoder
-    over an fp32 stream x (in place):
-        x += mult * RMSnorm(y_scale * (y + y2)) * w_post   (y given)
+                   add=None, pre_w=None, post_off: float = 0.0,
+                   pre_off: float = 0.0, cast=None):
+    """One launch per sublayer boundary of an RMS post- or sandwich-norm
+    decoder over an fp32 stream x (in place):
+        x += mult * RMSnorm(y_scale * (y + y2)) * (post_off + w_post)
+                                                           (y given)
         x += add                                           (add: fp32 [width])
-        returns RMSnorm(x) * pre_w in pre_w's dtype        (pre_w given)
+        returns RMSnorm(x) * (pre_off + pre_w) in pre_w's dtype
+                                                           (pre_w given)
+        or x itself in dtype ``cast``                      (cast given)
     y / y2 may be row views; statistics and sums are fp32."""
     if x.is_cuda:
         h = None
         if pre_w is not None:
-            h = torch.empty(x.shape, dtype=pre_w.dtype, device=x.device)
+            cast = pre_w.dtype
+        if cast is not None:
+            h = torch.empty(x.shape, dtype=cast, device=x.device)
         _seq_kernels().stream_rmsnorm(x, y, y2, w_post, add, h, pre_w,
                                       float(eps), float(mult),
-                                      float(y_scale))
+                                      float(y_scale), float(post_off),
+                                      float(pre_off))
         return h
     return torch_ref.stream_rmsnorm(x, y, w_post, eps, mult, y_scale, y2,
-                                    add, pre_w)
+                                    add, pre_w, post_off, pre_off, cast)
+
+
+def embed_rmsnorm(ids, positions, table, pos, w, scale: float,
+                  w_off: float, eps: float):
+    """Token embedding of a decoder that norms it: returns (x, h) with
+    x = RMSnorm(table[ids] * scale + pos[positions]) * (w_off + w) in fp32
+    (the residual stream) and h its copy in the table's dtype. ``pos``
+    (a learned position table) may be None."""
+    if table.is_cuda:
+        T, width = ids.shape[0], table.shape[1]
+        x = torch.empty(T, width, dtype=torch.float32, device=table.device)
+        h = torch.empty(T, width, dtype=table.dtype, device=table.device)
+        _seq_kernels().embed_rmsnorm(x, h, ids, positions, table, pos, w,
+                                     float(scale), float(w_off), float(eps))
+        return x, h
+    return torch_ref.embed_rmsnorm(ids, positions, table, pos, w, scale,
+                                   w_off, eps)
 
 
 def gated_act_mul(x: torch.Tensor, act: str = "silu") -> torch.Tensor:
@@ -918,6 +942,51 @@ def rms_weight_store(x, w, eps, cache=None, slot_mapping=None):
         _seq_kernels().rms_weight_store(out, x, w, eps, cache, slot_mapping)
         return out
     return torch_ref.rms_weight_store(x, w, eps, cache, slot_mapping)
+
+
+def latent_rope_store(q, ckv, w, eps, positions, slot_mapping, freqs, mag,
+                      cache, H, D, R, Dr) -> None:
+    """What a latent-attention layer prepares per token, in one launch:
+    cache row <- [RMSnorm(ckv[:R]) * w | ckv[R:] turned by the position],
+    and the last Dr columns of every head of q [T, H*(D+Dr)] turned in
+    place (pairs (2i, 2i+1), fp64 frequencies, cos / sin times mag)."""
+    if q.is_cuda:
+        _seq_kernels().latent_rope_store(q, ckv, w, float(eps), positions,
+                                         slot_mapping, freqs, float(mag),
+                                         cache, H, D, R, Dr)
+        return
+    torch_ref.latent_rope_store(q, ckv, w, eps, positions, slot_mapping,
+                                freqs, mag, cache, H, D, R, Dr)
+
+
+def latent_attention(q_lat, q_rot, cache, block_table, seq_lens,
+                     query_start_loc, scale, window=0, sinks=None,
+                     max_query_len=0) -> torch.Tensor:
+    """Ragged attention of H query heads over ONE cached row per token,
+    [latent (R) | rotated key part (Dr)] in ``cache`` [pages, page, 1,
+    R + Dr]: score = (q_lat . latent + q_rot . rotated) * scale, position
+    i sees 0 <= i - j < window (window <= 0: every j <= i), ``sinks``
+    (fp32 [H]) join the softmax denominator, and the result per head is
+    the weighted latent. q_lat [H, T, R], q_rot [T, H, Dr] (views are
+    fine); returns [H, T, R]."""
+    H, T, R = q_lat.shape
+    v_cache = cache[..., :R]
+    q = torch.cat([q_lat.transpose(0, 1), q_rot], -1).reshape(T, -1)
+    o = window_attention(q, None, cache, v_cache, block_table, seq_lens,
+                         query_start_loc, scale, window, 0, False,
+                         max_query_len, sinks=sinks)
+    return o.view(T, H, R).transpose(0, 1)
+
+
+def head_gate(x, gate=None) -> torch.Tensor:
+    """x [H, T, D] (head major) -> [T, H*D], each element times
+    sigmoid(gate [T, H*D]) when a gate is given (row views are fine)."""
+    H, T, D = x.shape
+    if x.is_cuda:
+        out = torch.empty(T, H * D, dtype=x.dtype, device=x.device)
+        _seq_kernels().head_gate(out, x, gate)
+        return out
+    return torch_ref.head_gate(x, gate)
 
 
 # --------------------------------------------------------------- streams
@@ -1076,6 +1145,24 @@ def relu2(x: torch.Tensor) -> torch.Tensor:
     return torch_ref.relu2(x)
 
 
+def gelu_erf(x: torch.Tensor) -> torch.Tensor:
+    """Exact gelu: z * Phi(z)."""
+    if x.is_cuda:
+        out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+        _seq_kernels().gelu_erf(out, x)
+        return out
+    return torch_ref.gelu_erf(x)
+
+
+def token_gate(z, table, ids, col0: int) -> torch.Tensor:
+    """gelu_tanh(z [T, n]) * table[ids, col0:col0 + n]."""
+    if z.is_cuda:
+        out = torch.empty(z.shape, dtype=z.dtype, device=z.device)
+        _seq_kernels().token_gate(out, z, table, ids, int(col0))
+        return out
+    return torch_ref.token_gate(z, table, ids, col0)
+
+
 # --------------------------------------------------------------- delta rule
 def causal_conv_silu(x, w, conv_state, slots, has_init, query_start_loc,
                      activation=True, max_query_len=0):
@@ -1159,6 +1246,33 @@ def general_delta_rule(r, k, v, w_logit, a_logit, w0, decay_scale, state,
     return gdn_ref.general_delta_rule(r, k, v, w_logit, a_logit, w0,
                                       decay_scale, state, slots, has_init,
                                       query_start_loc)
+
+
+def channel_delta_rule(q, k, v, a, b, A_log, dt_bias, state, slots,
+                       has_init, query_start_loc, q_scale,
+                       max_query_len=0) -> torch.Tensor:
+    """Ragged gated delta rule with a decay per (value head, key
+    channel), prompt portions and decode tokens in one launch. q, k
+    [T, G*Dk] raw (unit norms, q_scale, decays and write strengths are
+    formed in fp32 here), v [T, H*Dv], a [T, H*Dk] decay logits, b [T, H]
+    write-strength logits. Per head, g = exp(-exp(A_log) softplus(a +
+    dt_bias)), beta = sigmoid(b):
+        S <- diag(g) S;  S <- S + k (beta (v - S^T k))^T;  o = S^T q
+    fp32 state [slots, H, Dk, Dv] in place; returns fp32 [T, H, Dv].
+    ``max_query_len`` == 1 (decode-only batch) with Dv a multiple of 64
+    runs the one-token kernel; anything else stages token tiles in LDS."""
+    if q.is_cuda:
+        H, _, Dv = state.shape[1:]
+        o = torch.empty(q.shape[0], H, Dv, dtype=torch.float32,
+                        device=q.device)
+        _seq_kernels().channel_delta_rule(
+            o, q, k, v, a, b, A_log, dt_bias, state, slots, has_init,
+            query_start_loc, float(q_scale), int(max_query_len))
+        return o
+    from gllm_amd.ops import gdn_ref
+    return gdn_ref.channel_delta_rule(q, k, v, a, b, A_log, dt_bias, state,
+                                      slots, has_init, query_start_loc,
+                                      q_scale)
 
 
 def token_shift(h, mu, state, slots, has_init, query_start_loc,

@@ -29,6 +29,9 @@
 //                       optional fused sigmoid output gate
 //   rotate_scale_rows   turn the pairs of every head row by sign * pos * f
 //                       and scale (the inverse turn of rotated values)
+//   latent_rope_store   a latent-attention token: latent normed into its
+//                       cache row, the shared rotated key part behind it,
+//                       the query heads' rotated parts turned in place
 //   rms_weight_store    weighted RMS norm of a row, also scattered into a
 //                       single-head paged cache (a low-rank latent)
 //
@@ -288,7 +291,7 @@ __global__ __launch_bounds__(ATT_BLOCK) void window_attention_kernel(
     const int *__restrict__ seq_lens, const int *__restrict__ qsl, int B,
     int H, int G, int D, int Dv, int page, float scale, int window,
     int keep_first, int sink, const float *__restrict__ sinks,
-    float softcap) {
+    float softcap, long v_row, long v_head) {
   constexpr int PARTS = ATT_BLOCK / CT;
   constexpr int NC = 2;  // columns per thread when Dv > CT (Dv <= 512)
   extern __shared__ float smem[];
@@ -386,7 +389,7 @@ __global__ __launch_bounds__(ATT_BLOCK) void window_attention_kernel(
     for (int c = 0; c < NC; ++c) acc[c] *= corr;
     for (int jj = part; jj < n_tile; jj += PARTS) {
       const float pj = ps[jj];
-      const T *vr = v_cache + (rows[jj] * G + g) * Dv;
+      const T *vr = v_cache + rows[jj] * v_row + g * v_head;
 #pragma unroll
       for (int c = 0; c < NC; ++c) {
         const int d = col + c * CT;
@@ -577,8 +580,12 @@ void window_attention(torch::Tensor out, torch::Tensor q,
   TORCH_CHECK(rows_ok(q) && q.size(1) % D == 0);
   const int H = q.size(1) / D;
   TORCH_CHECK(H % G == 0, "query heads must be a multiple of kv heads");
-  TORCH_CHECK(k_cache.is_contiguous() && v_cache.is_contiguous() &&
-              k_cache.scalar_type() == st && v_cache.scalar_type() == st);
+  // the value rows may be a column block of the key rows (a cached latent
+  // whose first columns are the value)
+  TORCH_CHECK(k_cache.is_contiguous() && k_cache.scalar_type() == st &&
+              v_cache.scalar_type() == st && v_cache.stride(3) == 1 &&
+              v_cache.stride(0) == page * v_cache.stride(1) &&
+              (G == 1 || v_cache.stride(2) >= Dv));
   TORCH_CHECK(v_cache.size(0) == k_cache.size(0) && v_cache.size(1) == page &&
               v_cache.size(2) == G);
   TORCH_CHECK(rows_ok(out) && out.scalar_type() == st && out.size(0) == T &&
@@ -624,7 +631,8 @@ void window_attention(torch::Tensor out, torch::Tensor q,
                      seq_lens.data_ptr<int>(),                               \
                      query_start_loc.data_ptr<int>(), B, H, G, D, Dv, page,  \
                      (float)scale, (int)window, (int)keep_first,             \
-                     sink ? 1 : 0, sp, (float)softcap)
+                     sink ? 1 : 0, sp, (float)softcap,                       \
+                     (long)v_cache.stride(1), (long)v_cache.stride(2))
 #define RUN_CT(TT)                                                           \
   switch (ct) {                                                              \
     case 16: RUN(TT, 16); break;                                             \
@@ -747,7 +755,125 @@ __global__ __launch_bounds__(ATT_BLOCK) void rms_weight_store_kernel(
   }
 }
 
+// One workgroup per token, everything a latent-attention layer prepares:
+// the first R columns of the token's down projection are RMS normed and
+// stored in its cache row, the last Dr are turned by the token's position
+// and stored behind them, and the last Dr columns of every query head are
+// turned in place. The cos / sin table of the token is formed once.
+template <typename T>
+__global__ __launch_bounds__(ATT_BLOCK) void latent_rope_store_kernel(
+    T *__restrict__ q, long q_stride, const T *__restrict__ ckv,
+    long ckv_stride, const T *__restrict__ w, float eps,
+    const long *__restrict__ positions, const long *__restrict__ slot_mapping,
+    const double *__restrict__ freqs, float mag, T *__restrict__ cache, int H,
+    int D, int R, int Dr, int vec) {
+  extern __shared__ float cs_tab[];  // [Dr/2] cos, [Dr/2] sin
+  __shared__ float red[ATT_BLOCK / WAVE_SIZE];
+  const long t = blockIdx.x;
+  const int tid = threadIdx.x;
+  const int half = Dr / 2;
+  const double pos = (double)positions[t];
+  for (int p = tid; p < half; p += ATT_BLOCK) {
+    double sn, cs;
+    sincos(pos * freqs[p], &sn, &cs);
+    cs_tab[p] = (float)cs * mag;
+    cs_tab[half + p] = (float)sn * mag;
+  }
+  const T *src = ckv + t * ckv_stride;
+  T *crow = cache + slot_mapping[t] * (R + Dr);
+  float ss = 0.f;
+  if (vec) {
+    for (int i = tid * 8; i < R; i += ATT_BLOCK * 8) {
+      float f[8];
+      ld8<T>(src + i, f);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss += f[e] * f[e];
+    }
+  } else {
+    for (int i = tid; i < R; i += ATT_BLOCK) {
+      const float f = ScalarOps<T>::to_f32(src[i]);
+      ss += f * f;
+    }
+  }
+  // (the reduction's barriers also publish the cos / sin table)
+  const float inv =
+      1.0f / sqrtf(block_reduce_sum<ATT_BLOCK>(ss, red) / R + eps);
+  if (vec) {
+    for (int i = tid * 8; i < R; i += ATT_BLOCK * 8) {
+      float f[8], wf[8];
+      ld8<T>(src + i, f);
+      ld8<T>(w + i, wf);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) f[e] = f[e] * inv * wf[e];
+      st8<T>(crow + i, f);
+    }
+  } else {
+    for (int i = tid; i < R; i += ATT_BLOCK)
+      crow[i] = ScalarOps<T>::from_f32(ScalarOps<T>::to_f32(src[i]) * inv *
+                                       ScalarOps<T>::to_f32(w[i]));
+  }
+  // pair p of row y: y = H is the shared key part, y < H a query head
+  for (int idx = tid; idx < (H + 1) * half; idx += ATT_BLOCK) {
+    const int y = idx / half, p = idx % half;
+    T *qr = q + t * q_stride + (long)y * (D + Dr) + D + 2 * p;
+    const T *in = y == H ? src + R + 2 * p : qr;
+    T *dst = y == H ? crow + R + 2 * p : qr;
+    const float a = ScalarOps<T>::to_f32(in[0]);
+    const float b = ScalarOps<T>::to_f32(in[1]);
+    const float c = cs_tab[p], s = cs_tab[half + p];
+    dst[0] = ScalarOps<T>::from_f32(a * c - b * s);
+    dst[1] = ScalarOps<T>::from_f32(b * c + a * s);
+  }
+}
+
 }  // namespace
+
+void latent_rope_store(torch::Tensor q, torch::Tensor ckv, torch::Tensor w,
+                       double eps, torch::Tensor positions,
+                       torch::Tensor slot_mapping, torch::Tensor freqs,
+                       double mag, torch::Tensor cache, long H, long D,
+                       long R, long Dr) {
+  const long T = q.size(0);
+  if (T == 0) return;
+  const auto st = q.scalar_type();
+  TORCH_CHECK(q.is_cuda() && rows_ok(q) && q.size(1) == H * (D + Dr));
+  TORCH_CHECK(rows_ok(ckv) && ckv.size(0) == T && ckv.size(1) == R + Dr &&
+              ckv.scalar_type() == st);
+  TORCH_CHECK(w.scalar_type() == st && w.is_contiguous() && w.numel() == R);
+  TORCH_CHECK(positions.scalar_type() == at::kLong &&
+              positions.is_contiguous() && positions.numel() >= T);
+  TORCH_CHECK(slot_mapping.scalar_type() == at::kLong &&
+              slot_mapping.is_contiguous() && slot_mapping.numel() >= T);
+  TORCH_CHECK(Dr >= 0 && Dr % 2 == 0 && Dr <= 8192 &&
+              freqs.scalar_type() == at::kDouble && freqs.is_contiguous() &&
+              freqs.numel() * 2 >= Dr);
+  TORCH_CHECK(cache.is_contiguous() && cache.scalar_type() == st &&
+              cache.dim() == 4 && cache.size(2) == 1 &&
+              cache.size(3) == R + Dr,
+              "latent cache: [pages, page, 1, rank + rotated]");
+  const size_t es = q.element_size();
+  auto al16 = [&](const void *p, long stride) {
+    return reinterpret_cast<uintptr_t>(p) % 16 == 0 && (stride * es) % 16 == 0;
+  };
+  const bool vec = R % 8 == 0 && al16(ckv.data_ptr(), ckv.stride(0)) &&
+                   al16(w.data_ptr(), 0) && al16(cache.data_ptr(), R + Dr);
+  auto stream = at::cuda::getCurrentCUDAStream();
+#define RUN(TT)                                                              \
+  hipLaunchKernelGGL((latent_rope_store_kernel<TT>), dim3(T),                \
+                     dim3(ATT_BLOCK), Dr * sizeof(float), stream,            \
+                     (TT *)q.data_ptr(), (long)q.stride(0),                  \
+                     (const TT *)ckv.data_ptr(), (long)ckv.stride(0),        \
+                     (const TT *)w.data_ptr(), (float)eps,                   \
+                     positions.data_ptr<long>(),                             \
+                     slot_mapping.data_ptr<long>(), freqs.data_ptr<double>(), \
+                     (float)mag, (TT *)cache.data_ptr(), (int)H, (int)D,     \
+                     (int)R, (int)Dr, vec ? 1 : 0)
+  if (st == at::kBFloat16) RUN(__hip_bfloat16);
+  else if (st == at::kFloat) RUN(float);
+  else TORCH_CHECK(false, "latent_rope_store: bf16 or fp32");
+#undef RUN
+  HIP_CHECK_KERNEL();
+}
 
 void rotate_scale_rows(torch::Tensor out, torch::Tensor x,
                        torch::Tensor positions, torch::Tensor freqs,

@@ -107,7 +107,28 @@ void stream_rmsnorm(torch::Tensor x, c10::optional<torch::Tensor> y,
                     c10::optional<torch::Tensor> add,
                     c10::optional<torch::Tensor> h,
                     c10::optional<torch::Tensor> w_pre, double eps,
-                    double mult, double y_scale);
+                    double mult, double y_scale, double post_off,
+                    double pre_off);
+void embed_rmsnorm(torch::Tensor x, torch::Tensor h, torch::Tensor ids,
+                   torch::Tensor positions, torch::Tensor table,
+                   c10::optional<torch::Tensor> pos, torch::Tensor w,
+                   double scale, double w_off, double eps);
+void gelu_erf(torch::Tensor out, torch::Tensor x);
+void token_gate(torch::Tensor out, torch::Tensor z, torch::Tensor table,
+                torch::Tensor ids, long col0);
+void head_gate(torch::Tensor out, torch::Tensor x,
+               c10::optional<torch::Tensor> gate);
+void latent_rope_store(torch::Tensor q, torch::Tensor ckv, torch::Tensor w,
+                       double eps, torch::Tensor positions,
+                       torch::Tensor slot_mapping, torch::Tensor freqs,
+                       double mag, torch::Tensor cache, long H, long D,
+                       long R, long Dr);
+void channel_delta_rule(torch::Tensor o, torch::Tensor q, torch::Tensor k,
+                        torch::Tensor v, torch::Tensor a, torch::Tensor b,
+                        torch::Tensor A_log, torch::Tensor dt_bias,
+                        torch::Tensor state, torch::Tensor slots,
+                        torch::Tensor has_init, torch::Tensor query_start_loc,
+                        double q_scale, long max_query_len);
 void gated_act_mul(torch::Tensor out, torch::Tensor x, long act);
 void tanh_rows(torch::Tensor out, torch::Tensor x);
 void sigmoid_group_topk(torch::Tensor weights, torch::Tensor ids,
@@ -174,6 +195,18 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "ragged delta rule with per-channel decay and removal rate");
   m.def("stream_rmsnorm", &stream_rmsnorm,
         "x += mult * RMS(y) w_post (+ add); h = RMS(x) w_pre");
+  m.def("embed_rmsnorm", &embed_rmsnorm,
+        "x = RMS(table[id] * scale + pos[p]) * w and its model-dtype copy");
+  m.def("gelu_erf", &gelu_erf, "exact gelu over row-strided input");
+  m.def("token_gate", &token_gate,
+        "gelu_tanh(z) times a column block of a per-token table row");
+  m.def("head_gate", &head_gate,
+        "head-major heads to token-major rows, times sigmoid(gate)");
+  m.def("latent_rope_store", &latent_rope_store,
+        "latent norm + rotated key part into the paged cache, query heads' "
+        "rotated parts in place");
+  m.def("channel_delta_rule", &channel_delta_rule,
+        "ragged gated delta rule with a decay per key channel");
   m.def("gated_act_mul", &gated_act_mul, "act(x[:d]) * x[d:], silu or gelu");
   m.def("tanh_rows", &tanh_rows, "tanh over strided rows");
   m.def("sigmoid_group_topk", &sigmoid_group_topk,

@@ -31,6 +31,8 @@
 //                      ak = sigmoid(.) k / (|k|^2 + 1e-6) (removal rate on
 //                      the unit key, folded) from a per-token pre-pass;
 //                      same lane layout as delta_rule_varlen
+//   channel_delta_rule delta_rule_varlen with a decay per (value head, key
+//                      channel), g = exp(-exp(A_log_h) softplus(a + dt))
 //
 // State layouts: conv [slots, C, taps-1] (oldest first), recurrent
 // [slots, H, Dk, Dv] fp32.
@@ -866,6 +868,355 @@ __global__ __launch_bounds__(256) void general_delta_tiled_kernel(
   }
 }
 
+// ------------------------------------------------------------------
+// Delta rule with a decay per (value head, key channel), unit keys and
+// queries shared by a group of value heads:
+//   S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+//   g = exp(-exp(A_log_h) softplus(a + dt_bias)),  beta = sigmoid(b)
+//
+// What a token needs besides its raw rows, once instead of by every wave:
+//   scal[t] = [ik(G) | iq(G) | beta(H)]  (1/|k|, scale/|q|, write strength)
+//   gdec[t, h, i] = g                    (fp32)
+// grid (tokens, ceil(H / 4)), block 256: a wave per value head; the first
+// value head of a group also forms the group's two unit factors.
+DEV_INLINE float softplus_f(float z) {
+  return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void channel_delta_prep_kernel(
+    float *__restrict__ scal, float *__restrict__ gdec,
+    const T *__restrict__ q, const T *__restrict__ k, long qkv_stride,
+    const T *__restrict__ a, long a_stride, const T *__restrict__ bproj,
+    long b_stride, const float *__restrict__ A_log,
+    const float *__restrict__ dt_bias, int H, int G, int Dk, float q_scale) {
+  const long t = blockIdx.x;
+  const int lane = threadIdx.x & 63;
+  const int h = blockIdx.y * 4 + (threadIdx.x >> 6);
+  if (h >= H) return;  // (no barrier in this kernel)
+  float *sc = scal + t * (2 * G + H);
+  const float rate = expf(A_log[h]);
+  const T *ar = a + t * a_stride + (long)h * Dk;
+  float *gr = gdec + (t * H + h) * Dk;
+  for (int i = lane; i < Dk; i += 64)
+    gr[i] = expf(-rate * softplus_f(ScalarOps<T>::to_f32(ar[i]) +
+                                    dt_bias[(long)h * Dk + i]));
+  if (lane == 0)
+    sc[2 * G + h] =
+        1.0f / (1.0f + expf(-ScalarOps<T>::to_f32(bproj[t * b_stride + h])));
+  const int per = H / G;
+  if (h % per) return;
+  const int g = h / per;
+  float sk = 0.f, sq = 0.f;
+  for (int i = lane; i < Dk; i += 64) {
+    const float kv = ScalarOps<T>::to_f32(k[t * qkv_stride + (long)g * Dk + i]);
+    const float qv = ScalarOps<T>::to_f32(q[t * qkv_stride + (long)g * Dk + i]);
+    sk += kv * kv;
+    sq += qv * qv;
+  }
+  sk = wave_reduce_sum(sk);
+  sq = wave_reduce_sum(sq);
+  if (lane == 0) {
+    sc[g] = 1.0f / sqrtf(sk + 1e-6f);
+    sc[G + g] = q_scale / sqrtf(sq + 1e-6f);
+  }
+}
+
+// sum over the LPC (4 or 16) adjacent lanes that share a state column
+template <int LPC> DEV_INLINE float lanes_sum(float v) {
+  v = quad_sum(v);
+  if (LPC == 16) {
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(
+        0, __builtin_bit_cast(int, v), 0x141, 0xF, 0xF, true));  // half mirror
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(
+        0, __builtin_bit_cast(int, v), 0x140, 0xF, 0xF, true));  // mirror
+  }
+  return v;
+}
+
+// Walks a portion token by token. LPC adjacent lanes share a state column
+// and split the key axis into slices of KP (LPC 4: most columns per wave,
+// for batches that fill the chip; 16: a quarter of the work per token and
+// lane, for a few sequences, where the chain of tokens is what takes
+// time). The workgroup's waves share k, q and the decay row of their head:
+// tiles of TT tokens are staged once per workgroup in LDS as fp32, double
+// buffered. grid (B, H, ceil(Dv / (256 / LPC))), block 256.
+template <typename T, int KP, int LPC>
+__global__ __launch_bounds__(256) void channel_delta_tiled_kernel(
+    float *__restrict__ o, const T *__restrict__ q, const T *__restrict__ k,
+    const T *__restrict__ v, long qkv_stride, const float *__restrict__ scal,
+    const float *__restrict__ gdec, float *__restrict__ state,
+    const long *__restrict__ slots, const int *__restrict__ has_init,
+    const int *__restrict__ qsl, int H, int G, int Dk, int Dv) {
+  constexpr int TT = KP == 64 ? 4 : 8;    // tokens per tile
+  constexpr int CB = 256 / LPC;           // state columns per workgroup
+  constexpr int KPP = KP + 4;             // padded slice: no bank clash
+  constexpr int DKP = LPC * KP;           // padded key size
+  constexpr int ROW = LPC * KPP;          // one operand row in LDS
+  constexpr int TOK_F = 3 * ROW + CB + 4; // k | q | g | v | scalars
+  constexpr int PER = TT * DKP / 256;     // elements per thread and operand
+  constexpr int VPER = (TT * CB + 255) / 256;
+  static_assert(TT * DKP % 256 == 0, "whole staging rounds");
+  __shared__ __attribute__((aligned(16))) float lds[2][TT * TOK_F];
+
+  const int b = blockIdx.x, h = blockIdx.y;
+  const int tid = threadIdx.x;
+  const int vcol = tid / LPC;  // column inside the block
+  const int col = blockIdx.z * CB + vcol;
+  const int part = tid % LPC;
+  const int i0 = part * KP;
+  const int g = h / (H / G);
+  const int start = qsl[b], end = qsl[b + 1];
+  if (start >= end) return;
+  const bool live = col < Dv;
+  const int colc = live ? col : Dv - 1;  // clamp loads, mask stores
+  const int SW = 2 * G + H;
+
+  float *sp = state + ((long)slots[b] * H + h) * Dk * Dv;
+  float S[KP];
+  const bool init = has_init[b] != 0;
+#pragma unroll
+  for (int i = 0; i < KP; ++i)
+    S[i] = (init && i0 + i < Dk) ? sp[(long)(i0 + i) * Dv + colc] : 0.f;
+
+  T stg_k[PER], stg_q[PER], stg_v[VPER];
+  float stg_g[PER];
+  float stg_s = 0.f;
+  auto stage_load = [&](int tile0) {
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int idx = j * 256 + tid;
+      const int i = idx % DKP;
+      const long t = tile0 + idx / DKP;
+      const bool ok = i < Dk && t < end;
+      stg_k[j] = ok ? k[t * qkv_stride + (long)g * Dk + i]
+                    : ScalarOps<T>::from_f32(0.f);
+      stg_q[j] = ok ? q[t * qkv_stride + (long)g * Dk + i]
+                    : ScalarOps<T>::from_f32(0.f);
+      stg_g[j] = ok ? gdec[(t * H + h) * Dk + i] : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < VPER; ++j) {
+      const int idx = j * 256 + tid;
+      const int c = blockIdx.z * CB + idx % CB;
+      const long t = tile0 + idx / CB;
+      stg_v[j] = (idx < TT * CB && c < Dv && t < end)
+                     ? v[t * qkv_stride + (long)h * Dv + c]
+                     : ScalarOps<T>::from_f32(0.f);
+    }
+    if (tid < TT * 4 && (tid & 3) < 3) {
+      const int which = tid & 3;
+      const long t = tile0 + (tid >> 2) < end ? tile0 + (tid >> 2) : end - 1;
+      stg_s = scal[t * SW + (which == 0 ? g : which == 1 ? G + g : 2 * G + h)];
+    }
+  };
+  auto stage_store = [&](float *buf) {
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int idx = j * 256 + tid;
+      const int i = idx % DKP;
+      float *tok = buf + (idx / DKP) * TOK_F + (i / KP) * KPP + i % KP;
+      tok[0] = ScalarOps<T>::to_f32(stg_k[j]);
+      tok[ROW] = ScalarOps<T>::to_f32(stg_q[j]);
+      tok[2 * ROW] = stg_g[j];
+    }
+#pragma unroll
+    for (int j = 0; j < VPER; ++j) {
+      const int idx = j * 256 + tid;
+      if (idx < TT * CB)
+        buf[(idx / CB) * TOK_F + 3 * ROW + idx % CB] =
+            ScalarOps<T>::to_f32(stg_v[j]);
+    }
+    if (tid < TT * 4)
+      buf[(tid >> 2) * TOK_F + 3 * ROW + CB + (tid & 3)] = stg_s;
+  };
+
+  stage_load(start);
+  stage_store(lds[0]);
+  __syncthreads();
+  int cur = 0;
+  for (int tile0 = start; tile0 < end; tile0 += TT) {
+    const bool more = tile0 + TT < end;
+    if (more) stage_load(tile0 + TT);
+    const int n = end - tile0 < TT ? end - tile0 : TT;
+    const float *buf = lds[cur];
+    for (int tt = 0; tt < n; ++tt) {
+      const float *tok = buf + tt * TOK_F;
+      const floatx4 *kp4 = reinterpret_cast<const floatx4 *>(tok + part * KPP);
+      const floatx4 *qp4 =
+          reinterpret_cast<const floatx4 *>(tok + ROW + part * KPP);
+      const floatx4 *gp4 =
+          reinterpret_cast<const floatx4 *>(tok + 2 * ROW + part * KPP);
+      const float *sc = tok + 3 * ROW + CB;
+      const float vc = tok[3 * ROW + vcol];
+      const float ik = sc[0], iq = sc[1], beta = sc[2];
+      float kc[KP];
+      float d0 = 0.f, d1 = 0.f, d2 = 0.f, d3 = 0.f;  // 4 chains, not one
+#pragma unroll
+      for (int i = 0; i < KP; i += 4) {
+        const floatx4 kk = kp4[i / 4], gg = gp4[i / 4];
+        kc[i] = kk[0]; kc[i + 1] = kk[1]; kc[i + 2] = kk[2]; kc[i + 3] = kk[3];
+        S[i] *= gg[0];
+        S[i + 1] *= gg[1];
+        S[i + 2] *= gg[2];
+        S[i + 3] *= gg[3];
+        d0 += S[i] * kk[0];
+        d1 += S[i + 1] * kk[1];
+        d2 += S[i + 2] * kk[2];
+        d3 += S[i + 3] * kk[3];
+      }
+      const float d = lanes_sum<LPC>((d0 + d1) + (d2 + d3)) * ik;
+      const float c = beta * (vc - d) * ik;
+      float e0 = 0.f, e1 = 0.f, e2 = 0.f, e3 = 0.f;
+#pragma unroll
+      for (int i = 0; i < KP; i += 4) {
+        const floatx4 qq = qp4[i / 4];
+        S[i] += kc[i] * c;
+        S[i + 1] += kc[i + 1] * c;
+        S[i + 2] += kc[i + 2] * c;
+        S[i + 3] += kc[i + 3] * c;
+        e0 += S[i] * qq[0];
+        e1 += S[i + 1] * qq[1];
+        e2 += S[i + 2] * qq[2];
+        e3 += S[i + 3] * qq[3];
+      }
+      const float od = lanes_sum<LPC>((e0 + e1) + (e2 + e3)) * iq;
+      if (live && part == 0)
+        o[((long)(tile0 + tt) * H + h) * Dv + col] = od;
+    }
+    if (more) stage_store(lds[cur ^ 1]);
+    __syncthreads();
+    cur ^= 1;
+  }
+  if (live) {
+#pragma unroll
+    for (int i = 0; i < KP; ++i)
+      if (i0 + i < Dk) sp[(long)(i0 + i) * Dv + col] = S[i];
+  }
+}
+
+// One token per sequence (decode-only batches), Dv % 64 == 0. A workgroup
+// owns 64 state columns of a head: thread = (16 groups of 4 columns) x (16
+// key parts), rows part, part + 16, ..., so a wave's 16 B accesses cover
+// whole 256 B row segments of the state, which is read and written once.
+// Decay, write strength and the unit factors are formed here (no
+// pre-pass). grid (B, H, Dv / 64), block 256; Dk <= 16 * RP.
+template <typename T, int RP>
+__global__ __launch_bounds__(256) void channel_delta_decode_kernel(
+    float *__restrict__ o, const T *__restrict__ q, const T *__restrict__ k,
+    const T *__restrict__ v, long qkv_stride, const T *__restrict__ a,
+    long a_stride, const T *__restrict__ bproj, long b_stride,
+    const float *__restrict__ A_log, const float *__restrict__ dt_bias,
+    float *__restrict__ state, const long *__restrict__ slots,
+    const int *__restrict__ has_init, const int *__restrict__ qsl, int H,
+    int G, int Dk, int Dv, float q_scale) {
+  __shared__ float ks[16 * RP], qs[16 * RP], gs[16 * RP];
+  __shared__ __attribute__((aligned(16))) float red_d[4][64], red_o[4][64];
+  __shared__ float red_n[2][4];
+  const int b = blockIdx.x, h = blockIdx.y;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int c4 = (tid & 15) * 4, part = tid >> 4;
+  const int c0 = blockIdx.z * 64;
+  const int g = h / (H / G);
+  const long t = qsl[b];
+  if (qsl[b + 1] <= t) return;  // whole workgroup
+  float *sp = state + ((long)slots[b] * H + h) * Dk * Dv + c0 + c4;
+  const bool init = has_init[b] != 0;
+  floatx4 S[RP];
+#pragma unroll
+  for (int r = 0; r < RP; ++r) {
+    const int i = r * 16 + part;
+    S[r] = (init && i < Dk)
+               ? *reinterpret_cast<const floatx4 *>(sp + (long)i * Dv)
+               : floatx4{0.f, 0.f, 0.f, 0.f};
+  }
+  float vc[4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+    vc[e] = ScalarOps<T>::to_f32(
+        v[t * qkv_stride + (long)h * Dv + c0 + c4 + e]);
+  float sk = 0.f, sq = 0.f;
+  if (tid < 16 * RP) {  // RP <= 16: one key channel per thread
+    float kv = 0.f, qv = 0.f, gv = 0.f;
+    if (tid < Dk) {
+      kv = ScalarOps<T>::to_f32(k[t * qkv_stride + (long)g * Dk + tid]);
+      qv = ScalarOps<T>::to_f32(q[t * qkv_stride + (long)g * Dk + tid]);
+      gv = expf(-expf(A_log[h]) *
+                softplus_f(ScalarOps<T>::to_f32(
+                               a[t * a_stride + (long)h * Dk + tid]) +
+                           dt_bias[(long)h * Dk + tid]));
+    }
+    ks[tid] = kv;
+    qs[tid] = qv;
+    gs[tid] = gv;
+    sk = kv * kv;
+    sq = qv * qv;
+  }
+  sk = wave_reduce_sum(sk);
+  sq = wave_reduce_sum(sq);
+  if (lane == 0) {
+    red_n[0][wave] = sk;
+    red_n[1][wave] = sq;
+  }
+  const float beta =
+      1.0f / (1.0f + expf(-ScalarOps<T>::to_f32(bproj[t * b_stride + h])));
+  __syncthreads();
+  const float ik = 1.0f / sqrtf((red_n[0][0] + red_n[0][1]) +
+                                (red_n[0][2] + red_n[0][3]) + 1e-6f);
+  const float iq = q_scale / sqrtf((red_n[1][0] + red_n[1][1]) +
+                                   (red_n[1][2] + red_n[1][3]) + 1e-6f);
+  float d[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int r = 0; r < RP; ++r) {
+    const float gg = gs[r * 16 + part], kk = ks[r * 16 + part];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      S[r][e] *= gg;
+      d[e] += S[r][e] * kk;
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    d[e] += __shfl_xor(d[e], 16, 64);
+    d[e] += __shfl_xor(d[e], 32, 64);
+  }
+  if (lane < 16)
+    *reinterpret_cast<floatx4 *>(&red_d[wave][c4]) =
+        floatx4{d[0], d[1], d[2], d[3]};
+  __syncthreads();
+  float c[4], out[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const float dd = (red_d[0][c4 + e] + red_d[1][c4 + e]) +
+                     (red_d[2][c4 + e] + red_d[3][c4 + e]);
+    c[e] = beta * (vc[e] - dd * ik) * ik;
+  }
+#pragma unroll
+  for (int r = 0; r < RP; ++r) {
+    const int i = r * 16 + part;
+    const float kk = ks[i], qq = qs[i];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      S[r][e] += kk * c[e];
+      out[e] += S[r][e] * qq;
+    }
+    if (i < Dk) *reinterpret_cast<floatx4 *>(sp + (long)i * Dv) = S[r];
+  }
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    out[e] += __shfl_xor(out[e], 16, 64);
+    out[e] += __shfl_xor(out[e], 32, 64);
+  }
+  if (lane < 16)
+    *reinterpret_cast<floatx4 *>(&red_o[wave][c4]) =
+        floatx4{out[0], out[1], out[2], out[3]};
+  __syncthreads();
+  if (tid < 64)
+    o[(t * H + h) * Dv + c0 + tid] =
+        ((red_o[0][tid] + red_o[1][tid]) + (red_o[2][tid] + red_o[3][tid])) *
+        iq;
+}
+
 bool rows_ok(const torch::Tensor &t) {
   return t.dim() == 2 && t.stride(1) == 1;
 }
@@ -1270,5 +1621,113 @@ void general_delta_rule(torch::Tensor o, torch::Tensor r, torch::Tensor k,
 #undef RUN_KP
 #undef RUNT
 #undef RUN
+  HIP_CHECK_KERNEL();
+}
+
+void channel_delta_rule(torch::Tensor o, torch::Tensor q, torch::Tensor k,
+                        torch::Tensor v, torch::Tensor a, torch::Tensor b,
+                        torch::Tensor A_log, torch::Tensor dt_bias,
+                        torch::Tensor state, torch::Tensor slots,
+                        torch::Tensor has_init, torch::Tensor query_start_loc,
+                        double q_scale, long max_query_len) {
+  const long T = q.size(0);
+  if (T == 0) return;
+  const auto st = q.scalar_type();
+  TORCH_CHECK(q.is_cuda() && state.dim() == 4 &&
+              state.scalar_type() == at::kFloat && state.is_contiguous());
+  const int H = state.size(1), Dk = state.size(2), Dv = state.size(3);
+  TORCH_CHECK(rows_ok(q) && rows_ok(k) && rows_ok(v) && rows_ok(a) &&
+              rows_ok(b));
+  TORCH_CHECK(k.scalar_type() == st && v.scalar_type() == st &&
+              a.scalar_type() == st && b.scalar_type() == st);
+  TORCH_CHECK(q.size(1) % Dk == 0 && k.size(1) == q.size(1));
+  const int G = q.size(1) / Dk;
+  TORCH_CHECK(G > 0 && H % G == 0 && v.size(1) == (long)H * Dv);
+  TORCH_CHECK(q.stride(0) == k.stride(0) && q.stride(0) == v.stride(0),
+              "q, k, v must share a row stride (slices of one buffer)");
+  TORCH_CHECK(a.size(1) == (long)H * Dk && b.size(1) == H,
+              "channel_delta_rule: decay logits [T, H*Dk], b [T, H]");
+  TORCH_CHECK(k.size(0) == T && v.size(0) == T && a.size(0) == T &&
+              b.size(0) == T);
+  TORCH_CHECK(A_log.scalar_type() == at::kFloat && A_log.numel() == H &&
+              A_log.is_contiguous() && dt_bias.scalar_type() == at::kFloat &&
+              dt_bias.is_contiguous() && dt_bias.numel() == (long)H * Dk);
+  TORCH_CHECK(o.scalar_type() == at::kFloat && o.is_contiguous() &&
+              o.numel() == T * H * Dv);
+  const int B = slots.numel();
+  TORCH_CHECK(slots.scalar_type() == at::kLong && slots.is_contiguous());
+  TORCH_CHECK(has_init.scalar_type() == at::kInt && has_init.numel() == B);
+  TORCH_CHECK(query_start_loc.scalar_type() == at::kInt &&
+              query_start_loc.numel() >= B + 1);
+  TORCH_CHECK(Dk <= 256, "channel delta rule: key size <= 256");
+  TORCH_CHECK(st == at::kBFloat16 || st == at::kFloat,
+              "channel_delta_rule: bf16 or fp32");
+  auto stream = at::cuda::getCurrentCUDAStream();
+  if (max_query_len == 1 && T == B && Dv % 64 == 0 &&
+      reinterpret_cast<uintptr_t>(state.data_ptr()) % 16 == 0) {
+#define DEC(TT, RP)                                                          \
+  hipLaunchKernelGGL((channel_delta_decode_kernel<TT, RP>),                  \
+                     dim3(B, H, Dv / 64), dim3(256), 0, stream,              \
+                     o.data_ptr<float>(), (const TT *)q.data_ptr(),          \
+                     (const TT *)k.data_ptr(), (const TT *)v.data_ptr(),     \
+                     (long)q.stride(0), (const TT *)a.data_ptr(),            \
+                     (long)a.stride(0), (const TT *)b.data_ptr(),            \
+                     (long)b.stride(0), A_log.data_ptr<float>(),             \
+                     dt_bias.data_ptr<float>(), state.data_ptr<float>(),     \
+                     slots.data_ptr<long>(), has_init.data_ptr<int>(),       \
+                     query_start_loc.data_ptr<int>(), H, G, Dk, Dv,          \
+                     (float)q_scale)
+#define DEC_RP(TT)                                                           \
+  if (Dk <= 64) DEC(TT, 4);                                                  \
+  else if (Dk <= 128) DEC(TT, 8);                                            \
+  else DEC(TT, 16)
+    if (st == at::kBFloat16) { DEC_RP(__hip_bfloat16); }
+    else { DEC_RP(float); }
+#undef DEC_RP
+#undef DEC
+    HIP_CHECK_KERNEL();
+    return;
+  }
+  auto fopt = o.options().dtype(at::kFloat);
+  auto scal = torch::empty({T, 2 * G + H}, fopt);
+  auto gdec = torch::empty({T, H, Dk}, fopt);
+#define PREP(TT)                                                             \
+  hipLaunchKernelGGL((channel_delta_prep_kernel<TT>), dim3(T, (H + 3) / 4),  \
+                     dim3(256), 0, stream, scal.data_ptr<float>(),           \
+                     gdec.data_ptr<float>(), (const TT *)q.data_ptr(),       \
+                     (const TT *)k.data_ptr(), (long)q.stride(0),            \
+                     (const TT *)a.data_ptr(), (long)a.stride(0),            \
+                     (const TT *)b.data_ptr(), (long)b.stride(0),            \
+                     A_log.data_ptr<float>(), dt_bias.data_ptr<float>(), H,  \
+                     G, Dk, (float)q_scale)
+  if (st == at::kBFloat16) PREP(__hip_bfloat16);
+  else PREP(float);
+#undef PREP
+  // a few sequences leave most of the chip idle at 64 columns a workgroup:
+  // sixteen lanes per column then shorten every token's chain
+  const bool wide = Dk > 32 && (long)B * H * ((Dv + 63) / 64) < 512;
+#define RUNT(TT, KPV, L)                                                     \
+  hipLaunchKernelGGL((channel_delta_tiled_kernel<TT, KPV, L>),               \
+                     dim3(B, H, (Dv + 256 / L - 1) / (256 / L)), dim3(256),  \
+                     0, stream, o.data_ptr<float>(),                         \
+                     (const TT *)q.data_ptr(), (const TT *)k.data_ptr(),     \
+                     (const TT *)v.data_ptr(), (long)q.stride(0),            \
+                     scal.data_ptr<float>(), gdec.data_ptr<float>(),         \
+                     state.data_ptr<float>(), slots.data_ptr<long>(),        \
+                     has_init.data_ptr<int>(),                               \
+                     query_start_loc.data_ptr<int>(), H, G, Dk, Dv)
+#define RUN_KP(TT)                                                           \
+  if (Dk <= 32) RUNT(TT, 8, 4);                                              \
+  else if (wide) {                                                           \
+    if (Dk <= 64) RUNT(TT, 4, 16);                                           \
+    else if (Dk <= 128) RUNT(TT, 8, 16);                                     \
+    else RUNT(TT, 16, 16);                                                   \
+  } else if (Dk <= 64) RUNT(TT, 16, 4);                                      \
+  else if (Dk <= 128) RUNT(TT, 32, 4);                                       \
+  else RUNT(TT, 64, 4)
+  if (st == at::kBFloat16) { RUN_KP(__hip_bfloat16); }
+  else { RUN_KP(float); }
+#undef RUN_KP
+#undef RUNT
   HIP_CHECK_KERNEL();
 }

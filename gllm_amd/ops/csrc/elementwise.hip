@@ -270,6 +270,13 @@ struct Relu2Op {
   }
 };
 
+struct GeluErfOp {
+  // z Phi(z)
+  DEV_INLINE float operator()(float z) const {
+    return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f));
+  }
+};
+
 template <typename T, typename Op, bool VEC>
 __global__ __launch_bounds__(256) void unary_rows_kernel(
     T *__restrict__ out, const T *__restrict__ x, long x_stride, long rows,
@@ -340,6 +347,169 @@ void xielu(torch::Tensor out, torch::Tensor x, double a_pos, double a_neg) {
 
 void relu2(torch::Tensor out, torch::Tensor x) {
   launch_unary_rows(out, x, Relu2Op{}, "relu2");
+}
+
+void gelu_erf(torch::Tensor out, torch::Tensor x) {
+  launch_unary_rows(out, x, GeluErfOp{}, "gelu_erf");
+}
+
+namespace {
+
+// out[r, i] = gelu_tanh(z[r, i]) * table[ids[r], col0 + i]: a per-token
+// table row gates a low-width projection. Ids are clamped to the table.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void token_gate_kernel(
+    T *__restrict__ out, const T *__restrict__ z, long z_stride,
+    const T *__restrict__ table, long t_stride, long n_vocab,
+    const long *__restrict__ ids, long rows, int n, int col0) {
+  constexpr int E = VEC ? 8 : 1;
+  const int nv = n / E;
+  const long total = rows * nv;
+  for (long idx = blockIdx.x * (long)blockDim.x + threadIdx.x; idx < total;
+       idx += (long)gridDim.x * blockDim.x) {
+    const long r = idx / nv;
+    const int i = (idx % nv) * E;
+    long id = ids[r];
+    id = id < 0 ? 0 : id < n_vocab ? id : n_vocab - 1;
+    const T *zr = z + r * z_stride + i;
+    const T *er = table + id * t_stride + col0 + i;
+    float f[E], e[E];
+    if (VEC) {
+      ld8<T>(zr, f);
+      ld8<T>(er, e);
+    } else {
+      f[0] = ScalarOps<T>::to_f32(zr[0]);
+      e[0] = ScalarOps<T>::to_f32(er[0]);
+    }
+#pragma unroll
+    for (int j = 0; j < E; ++j) {
+      const float v = f[j];
+      const float u = 0.79788456080286536f * (v + 0.044715f * v * v * v);
+      f[j] = 0.5f * v * (1.0f + tanhf(u)) * e[j];
+    }
+    if (VEC) st8<T>(out + r * n + i, f);
+    else out[r * n + i] = ScalarOps<T>::from_f32(f[0]);
+  }
+}
+
+// head-major heads x [H, T, D] -> token-major rows out [T, H * D], each
+// element times sigmoid(gate[t, h * D + d]) when a gate is given
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void head_gate_kernel(
+    T *__restrict__ out, long out_stride, const T *__restrict__ x,
+    long x_hs, long x_ts, const T *__restrict__ gate, long g_stride, long rows,
+    int H, int D) {
+  constexpr int E = VEC ? 8 : 1;
+  const int nd = D / E, nv = H * nd;
+  const long total = rows * nv;
+  for (long idx = blockIdx.x * (long)blockDim.x + threadIdx.x; idx < total;
+       idx += (long)gridDim.x * blockDim.x) {
+    const long t = idx / nv;
+    const int w = idx % nv;
+    const int h = w / nd, d = (w % nd) * E;
+    const T *xr = x + h * x_hs + t * x_ts + d;
+    float f[E], z[E];
+    if (VEC) ld8<T>(xr, f);
+    else f[0] = ScalarOps<T>::to_f32(xr[0]);
+    if (gate) {
+      const T *gr = gate + t * g_stride + (long)h * D + d;
+      if (VEC) ld8<T>(gr, z);
+      else z[0] = ScalarOps<T>::to_f32(gr[0]);
+#pragma unroll
+      for (int j = 0; j < E; ++j) f[j] *= 1.0f / (1.0f + expf(-z[j]));
+    }
+    T *dst = out + t * out_stride + (long)h * D + d;
+    if (VEC) st8<T>(dst, f);
+    else dst[0] = ScalarOps<T>::from_f32(f[0]);
+  }
+}
+
+bool on16(const void *p, long stride, size_t es) {
+  return reinterpret_cast<uintptr_t>(p) % 16 == 0 && (stride * es) % 16 == 0;
+}
+
+}  // namespace
+
+void token_gate(torch::Tensor out, torch::Tensor z, torch::Tensor table,
+                torch::Tensor ids, long col0) {
+  const long rows = z.size(0);
+  const int n = z.size(1);
+  if (rows == 0 || n == 0) return;
+  const auto st = z.scalar_type();
+  TORCH_CHECK(z.is_cuda() && z.dim() == 2 && z.stride(1) == 1 &&
+              out.is_contiguous() && out.numel() == rows * n &&
+              out.scalar_type() == st);
+  TORCH_CHECK(table.dim() == 2 && table.stride(1) == 1 &&
+              table.scalar_type() == st && table.size(0) > 0 && col0 >= 0 &&
+              col0 + n <= table.size(1), "token_gate: table columns");
+  TORCH_CHECK(ids.scalar_type() == at::kLong && ids.is_contiguous() &&
+              ids.numel() >= rows);
+  const size_t es = z.element_size();
+  const bool vec = n % 8 == 0 && (col0 * es) % 16 == 0 &&
+                   on16(z.data_ptr(), z.stride(0), es) &&
+                   on16(table.data_ptr(), table.stride(0), es) &&
+                   on16(out.data_ptr(), n, es);
+  const long work = vec ? rows * (n / 8) : rows * (long)n;
+  const int grid = (int)std::min<long>((work + 255) / 256, 65535);
+  auto stream = at::cuda::getCurrentCUDAStream();
+#define RUN(TT, V)                                                          \
+  hipLaunchKernelGGL((token_gate_kernel<TT, V>), dim3(grid), dim3(256), 0,  \
+                     stream, (TT *)out.data_ptr(), (const TT *)z.data_ptr(), \
+                     (long)z.stride(0), (const TT *)table.data_ptr(),       \
+                     (long)table.stride(0), (long)table.size(0),            \
+                     ids.data_ptr<long>(), rows, n, (int)col0)
+  if (st == at::kBFloat16) {
+    if (vec) RUN(__hip_bfloat16, true); else RUN(__hip_bfloat16, false);
+  } else if (st == at::kFloat) {
+    if (vec) RUN(float, true); else RUN(float, false);
+  } else {
+    TORCH_CHECK(false, "token_gate: bf16 or fp32");
+  }
+#undef RUN
+  HIP_CHECK_KERNEL();
+}
+
+void head_gate(torch::Tensor out, torch::Tensor x,
+               c10::optional<torch::Tensor> gate) {
+  const int H = x.size(0), D = x.size(2);
+  const long rows = x.size(1);
+  if (rows == 0) return;
+  const auto st = x.scalar_type();
+  TORCH_CHECK(x.is_cuda() && x.dim() == 3 && x.stride(2) == 1,
+              "head_gate: x [H, T, D]");
+  TORCH_CHECK(out.dim() == 2 && out.stride(1) == 1 && out.size(0) == rows &&
+              out.size(1) == (long)H * D && out.scalar_type() == st);
+  const size_t es = x.element_size();
+  bool vec = D % 8 == 0 && on16(x.data_ptr(), x.stride(0), es) &&
+             (x.stride(1) * es) % 16 == 0 &&
+             on16(out.data_ptr(), out.stride(0), es);
+  const void *gp = nullptr;
+  long gs = 0;
+  if (gate.has_value()) {
+    TORCH_CHECK(gate->dim() == 2 && gate->stride(1) == 1 &&
+                gate->size(0) == rows && gate->size(1) == (long)H * D &&
+                gate->scalar_type() == st);
+    gp = gate->data_ptr();
+    gs = gate->stride(0);
+    vec = vec && on16(gp, gs, es);
+  }
+  const long work = rows * H * (vec ? D / 8 : D);
+  const int grid = (int)std::min<long>((work + 255) / 256, 65535);
+  auto stream = at::cuda::getCurrentCUDAStream();
+#define RUN(TT, V)                                                          \
+  hipLaunchKernelGGL((head_gate_kernel<TT, V>), dim3(grid), dim3(256), 0,   \
+                     stream, (TT *)out.data_ptr(), (long)out.stride(0),     \
+                     (const TT *)x.data_ptr(), (long)x.stride(0),           \
+                     (long)x.stride(1), (const TT *)gp, gs, rows, H, D)
+  if (st == at::kBFloat16) {
+    if (vec) RUN(__hip_bfloat16, true); else RUN(__hip_bfloat16, false);
+  } else if (st == at::kFloat) {
+    if (vec) RUN(float, true); else RUN(float, false);
+  } else {
+    TORCH_CHECK(false, "head_gate: bf16 or fp32");
+  }
+#undef RUN
+  HIP_CHECK_KERNEL();
 }
 
 namespace {

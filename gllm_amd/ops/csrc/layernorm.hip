@@ -9,7 +9,11 @@
 //                       with a gate: LN_post sees y * sigmoid(gate)
 //   stream_rmsnorm:     the RMS form (plain weight, eps inside the root,
 //                       no mean): x += mult * RMS(s (y + y2)) w_post;
-//                       x += add; h = RMS(x) w_pre — every part optional
+//                       x += add; h = RMS(x) w_pre — every part optional;
+//                       weights may be stored as their distance from an
+//                       offset; without w_pre h is x in the model dtype
+//   embed_rmsnorm:      x = RMS(table[id] scale + pos[p]) w, the stream
+//                       of a decoder that norms its embedding
 //
 // One workgroup per token row; the row lives in LDS as fp32 between the
 // mean, variance (mean of squared deviations, two passes: no E[x^2] -
@@ -402,7 +406,7 @@ __global__ __launch_bounds__(LN_BLOCK) void stream_rmsnorm_kernel(
     const T *__restrict__ y2, long y2_stride, const T *__restrict__ w_post,
     const float *__restrict__ add, T *__restrict__ h,
     const T *__restrict__ w_pre, float eps, float mult, float y_scale,
-    int width, int vec) {
+    float post_off, float pre_off, int width, int vec) {
   extern __shared__ float row[];
   __shared__ float red[LN_BLOCK / WAVE_SIZE];
   const long base = (long)blockIdx.x * width;
@@ -447,7 +451,7 @@ __global__ __launch_bounds__(LN_BLOCK) void stream_rmsnorm_kernel(
         if (add) ld8<float>(add + i, af);
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-          xf[e] += row[i + e] * inv * wf[e];
+          xf[e] += row[i + e] * inv * (post_off + wf[e]);
           xf[e] += af[e];
           row[i + e] = xf[e];
           ss += xf[e] * xf[e];
@@ -456,7 +460,8 @@ __global__ __launch_bounds__(LN_BLOCK) void stream_rmsnorm_kernel(
       }
     } else {
       for (int i = tid; i < width; i += LN_BLOCK) {
-        float r = x[base + i] + row[i] * inv * ScalarOps<T>::to_f32(w_post[i]);
+        float r = x[base + i] +
+                  row[i] * inv * (post_off + ScalarOps<T>::to_f32(w_post[i]));
         if (add) r += add[i];
         x[base + i] = r;
         row[i] = r;
@@ -493,19 +498,97 @@ __global__ __launch_bounds__(LN_BLOCK) void stream_rmsnorm_kernel(
     }
   }
   if (h == nullptr) return;
+  if (w_pre == nullptr) {  // the next sublayer reads the stream itself
+    if (vec) {
+      for (int i = tid * 8; i < width; i += LN_BLOCK * 8)
+        st8<T>(h + base + i, row + i);
+    } else {
+      for (int i = tid; i < width; i += LN_BLOCK)
+        h[base + i] = ScalarOps<T>::from_f32(row[i]);
+    }
+    return;
+  }
   const float inv = 1.0f / sqrtf(ln_block_sum(ss, red) / width + eps);
   if (vec) {
     for (int i = tid * 8; i < width; i += LN_BLOCK * 8) {
       float wf[8], of[8];
       ld8<T>(w_pre + i, wf);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) of[e] = row[i + e] * inv * wf[e];
+      for (int e = 0; e < 8; ++e)
+        of[e] = row[i + e] * inv * (pre_off + wf[e]);
       st8<T>(h + base + i, of);
     }
   } else {
     for (int i = tid; i < width; i += LN_BLOCK)
-      h[base + i] = ScalarOps<T>::from_f32(row[i] * inv *
-                                           ScalarOps<T>::to_f32(w_pre[i]));
+      h[base + i] = ScalarOps<T>::from_f32(
+          row[i] * inv * (pre_off + ScalarOps<T>::to_f32(w_pre[i])));
+  }
+}
+
+// Token embedding of a decoder whose stream opens with a norm:
+//   r = table[id] * scale + pos[p];  x = r / rms(r) * (w_off + w)
+// x fp32, h = x in the model dtype (what the first sublayer reads).
+// Ids and positions are clamped to their tables (padding rows of a
+// profile pass carry any position). grid (tokens), one row in LDS.
+template <typename T>
+__global__ __launch_bounds__(LN_BLOCK) void embed_rmsnorm_kernel(
+    float *__restrict__ x, T *__restrict__ h, const long *__restrict__ ids,
+    const long *__restrict__ positions, const T *__restrict__ table,
+    long n_vocab, const T *__restrict__ pos, long n_pos,
+    const T *__restrict__ w, float scale, float w_off, float eps, int width,
+    int vec) {
+  extern __shared__ float row[];
+  __shared__ float red[LN_BLOCK / WAVE_SIZE];
+  const int tid = threadIdx.x;
+  const long base = (long)blockIdx.x * width;
+  long id = ids[blockIdx.x];
+  id = id < 0 ? 0 : id < n_vocab ? id : n_vocab - 1;
+  const T *src = table + id * width;
+  const T *ps = nullptr;
+  if (pos) {
+    long p = positions[blockIdx.x];
+    p = p < 0 ? 0 : p < n_pos ? p : n_pos - 1;
+    ps = pos + p * width;
+  }
+  float ss = 0.f;
+  if (vec) {
+    for (int i = tid * 8; i < width; i += LN_BLOCK * 8) {
+      float a[8], b[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      ld8<T>(src + i, a);
+      if (ps) ld8<T>(ps + i, b);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        a[e] = a[e] * scale + b[e];
+        row[i + e] = a[e];
+        ss += a[e] * a[e];
+      }
+    }
+  } else {
+    for (int i = tid; i < width; i += LN_BLOCK) {
+      float a = ScalarOps<T>::to_f32(src[i]) * scale;
+      if (ps) a += ScalarOps<T>::to_f32(ps[i]);
+      row[i] = a;
+      ss += a * a;
+    }
+  }
+  const float inv = 1.0f / sqrtf(ln_block_sum(ss, red) / width + eps);
+  // each thread revisits exactly the elements it wrote above
+  if (vec) {
+    for (int i = tid * 8; i < width; i += LN_BLOCK * 8) {
+      float wf[8];
+      ld8<T>(w + i, wf);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) wf[e] = row[i + e] * inv * (w_off + wf[e]);
+      st8<float>(x + base + i, wf);
+      st8<T>(h + base + i, wf);
+    }
+  } else {
+    for (int i = tid; i < width; i += LN_BLOCK) {
+      const float v =
+          row[i] * inv * (w_off + ScalarOps<T>::to_f32(w[i]));
+      x[base + i] = v;
+      h[base + i] = ScalarOps<T>::from_f32(v);
+    }
   }
 }
 
@@ -517,7 +600,8 @@ void stream_rmsnorm(torch::Tensor x, c10::optional<torch::Tensor> y,
                     c10::optional<torch::Tensor> add,
                     c10::optional<torch::Tensor> h,
                     c10::optional<torch::Tensor> w_pre, double eps,
-                    double mult, double y_scale) {
+                    double mult, double y_scale, double post_off,
+                    double pre_off) {
   TORCH_CHECK(x.is_cuda() && x.scalar_type() == at::kFloat &&
               x.is_contiguous());
   const int width = x.size(-1);
@@ -561,13 +645,15 @@ void stream_rmsnorm(torch::Tensor x, c10::optional<torch::Tensor> y,
     vec = vec && aligned16(addp);
   }
   if (h.has_value()) {
-    TORCH_CHECK(w_pre.has_value());
     TORCH_CHECK(h->is_contiguous() && h->numel() == x.numel() &&
                 h->scalar_type() == st);
-    check_vec(*w_pre, width, st);
     hp = h->data_ptr();
-    wpre = w_pre->data_ptr();
-    vec = vec && aligned16(hp) && aligned16(wpre);
+    vec = vec && aligned16(hp);
+    if (w_pre.has_value()) {  // none: h is the stream in its own dtype
+      check_vec(*w_pre, width, st);
+      wpre = w_pre->data_ptr();
+      vec = vec && aligned16(wpre);
+    }
   }
   auto stream = at::cuda::getCurrentCUDAStream();
 #define RUN(T)                                                              \
@@ -575,11 +661,59 @@ void stream_rmsnorm(torch::Tensor x, c10::optional<torch::Tensor> y,
                      width * sizeof(float), stream, x.data_ptr<float>(),    \
                      (const T *)yp, ys, (const T *)y2p, y2s,                \
                      (const T *)wpost, addp, (T *)hp, (const T *)wpre,      \
-                     (float)eps, (float)mult, (float)y_scale, width,        \
-                     vec ? 1 : 0)
+                     (float)eps, (float)mult, (float)y_scale,               \
+                     (float)post_off, (float)pre_off, width, vec ? 1 : 0)
   if (st == at::kBFloat16) RUN(__hip_bfloat16);
   else if (st == at::kFloat) RUN(float);
   else TORCH_CHECK(false, "stream_rmsnorm: bf16 or fp32");
+#undef RUN
+  HIP_CHECK_KERNEL();
+}
+
+void embed_rmsnorm(torch::Tensor x, torch::Tensor h, torch::Tensor ids,
+                   torch::Tensor positions, torch::Tensor table,
+                   c10::optional<torch::Tensor> pos, torch::Tensor w,
+                   double scale, double w_off, double eps) {
+  const long rows = ids.numel();
+  if (rows == 0) return;
+  const auto st = h.scalar_type();
+  const int width = table.size(1);
+  TORCH_CHECK(x.is_cuda() && x.scalar_type() == at::kFloat &&
+              x.is_contiguous() && x.numel() == rows * width);
+  TORCH_CHECK(h.is_contiguous() && h.numel() == rows * width);
+  TORCH_CHECK(ids.scalar_type() == at::kLong && ids.is_contiguous());
+  TORCH_CHECK(table.dim() == 2 && table.is_contiguous() &&
+              table.scalar_type() == st && table.size(0) > 0);
+  TORCH_CHECK(width > 0 && width * 4 <= 64 * 1024);
+  check_vec(w, width, st);
+  const void *pp = nullptr;
+  long n_pos = 0;
+  bool vec = width % 8 == 0 && aligned16(x.data_ptr()) &&
+             aligned16(h.data_ptr()) && aligned16(table.data_ptr()) &&
+             aligned16(w.data_ptr());
+  if (pos.has_value()) {
+    TORCH_CHECK(pos->dim() == 2 && pos->is_contiguous() &&
+                pos->size(1) == width && pos->scalar_type() == st &&
+                pos->size(0) > 0);
+    TORCH_CHECK(positions.scalar_type() == at::kLong &&
+                positions.is_contiguous() && positions.numel() >= rows);
+    pp = pos->data_ptr();
+    n_pos = pos->size(0);
+    vec = vec && aligned16(pp);
+  }
+  auto stream = at::cuda::getCurrentCUDAStream();
+#define RUN(T)                                                              \
+  hipLaunchKernelGGL((embed_rmsnorm_kernel<T>), dim3(rows), dim3(LN_BLOCK), \
+                     width * sizeof(float), stream, x.data_ptr<float>(),    \
+                     (T *)h.data_ptr(), ids.data_ptr<long>(),               \
+                     pp ? positions.data_ptr<long>() : nullptr,             \
+                     (const T *)table.data_ptr(), (long)table.size(0),      \
+                     (const T *)pp, n_pos, (const T *)w.data_ptr(),         \
+                     (float)scale, (float)w_off, (float)eps, width,         \
+                     vec ? 1 : 0)
+  if (st == at::kBFloat16) RUN(__hip_bfloat16);
+  else if (st == at::kFloat) RUN(float);
+  else TORCH_CHECK(false, "embed_rmsnorm: bf16 or fp32");
 #undef RUN
   HIP_CHECK_KERNEL();
 }

@@ -332,3 +332,41 @@ def general_delta_rule(r, k, v, w_logit, a_logit, w0, decay_scale, state,
             out[t] = torch.einsum("hkv,hk->hv", S, rf[t])
         state[slot] = S
     return out
+
+
+def channel_delta_rule(q, k, v, a, b, A_log, dt_bias, state, slots,
+                       has_init, query_start_loc, q_scale):
+    """Token-by-token gated delta rule with a decay per (value head, key
+    channel) over a ragged batch; fp32 state [slots, H, Dk, Dv] in place.
+    q, k [T, G*Dk] raw, v [T, H*Dv], a [T, H*Dk], b [T, H], A_log [H],
+    dt_bias [H*Dk]; returns fp32 [T, H, Dv]."""
+    H, Dk, Dv = state.shape[1:]
+    T = q.shape[0]
+    G = q.shape[1] // Dk
+
+    def unit(x):
+        x = x.float().reshape(T, G, Dk)
+        x = x / torch.sqrt((x * x).sum(-1, keepdim=True) + 1e-6)
+        return x.repeat_interleave(H // G, dim=1)
+
+    qf, kf = unit(q) * q_scale, unit(k)
+    vf = v.float().reshape(T, H, Dv)
+    decay = torch.exp(-torch.exp(A_log.float())[:, None] *
+                      torch.nn.functional.softplus(
+                          a.float() + dt_bias.float()).reshape(T, H, Dk))
+    beta = torch.sigmoid(b.float())
+    out = torch.empty(T, H, Dv, dtype=torch.float32)
+    qsl = query_start_loc.tolist()
+    for i, slot in enumerate(slots.tolist()):
+        if qsl[i + 1] <= qsl[i]:
+            continue
+        S = state[slot].clone() if bool(has_init[i]) \
+            else torch.zeros(H, Dk, Dv)
+        for t in range(qsl[i], qsl[i + 1]):
+            S = S * decay[t, :, :, None]
+            d = torch.einsum("hkv,hk->hv", S, kf[t])
+            u = beta[t][:, None] * (vf[t] - d)
+            S = S + kf[t][:, :, None] * u[:, None, :]
+            out[t] = torch.einsum("hkv,hk->hv", S, qf[t])
+        state[slot] = S
+    return out

@@ -289,24 +289,38 @@ def residual_layernorm(x: torch.Tensor, y: torch.Tensor, w_post, b_post,
 
 
 def stream_rmsnorm(x, y, w_post, eps, mult=1.0, y_scale=1.0, y2=None,
-                   add=None, pre_w=None):
+                   add=None, pre_w=None, post_off=0.0, pre_off=0.0,
+                   cast=None):
     """fp32 stream x (in place): x += mult * RMSnorm(y_scale * (y + y2))
-    * w_post (skipped when ``y`` is None), then x += add (one fp32 row
-    for every token); returns RMSnorm(x) * pre_w in pre_w's dtype when
-    ``pre_w`` is given."""
+    * (post_off + w_post) (skipped when ``y`` is None), then x += add (one
+    fp32 row for every token); returns RMSnorm(x) * (pre_off + pre_w) in
+    pre_w's dtype when ``pre_w`` is given, else x in dtype ``cast`` when
+    that is given."""
     if y is not None:
         z = y.float()
         if y2 is not None:
             z = z + y2.float()
         z = z * y_scale
         z = z * torch.rsqrt((z * z).mean(-1, keepdim=True) + eps)
-        x.add_(z * w_post.float() * mult)
+        x.add_(z * (post_off + w_post.float()) * mult)
     if add is not None:
         x.add_(add.float())
     if pre_w is None:
-        return None
+        # a copy: the caller goes on adding to x
+        return None if cast is None else x.to(cast, copy=True)
     h = x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps)
-    return (h * pre_w.float()).to(pre_w.dtype)
+    return (h * (pre_off + pre_w.float())).to(pre_w.dtype)
+
+
+def embed_rmsnorm(ids, positions, table, pos, w, scale, w_off, eps):
+    """(x, h): x = RMSnorm(table[ids] * scale + pos[positions]) *
+    (w_off + w) in fp32, h = x in the table's dtype."""
+    r = table[ids].float() * scale
+    if pos is not None:
+        r = r + pos[positions.clamp(0, pos.shape[0] - 1)].float()
+    x = r * torch.rsqrt((r * r).mean(-1, keepdim=True) + eps) \
+        * (w_off + w.float())
+    return x, x.to(table.dtype, copy=True)
 
 
 def token_shift(h, mu, state, slots, has_init, query_start_loc):
@@ -465,6 +479,39 @@ def rms_weight_store(x, w, eps, cache=None, slot_mapping=None):
         cache.view(-1, x.shape[1])[slot_mapping[:x.shape[0]]] = \
             y.to(cache.dtype)
     return y
+
+
+def latent_rope_store(q, ckv, w, eps, positions, slot_mapping, freqs, mag,
+                      cache, H, D, R, Dr):
+    """Latent normed + rotated key part into the paged cache; the query
+    heads' rotated parts (last Dr of D + Dr) turned in place."""
+    T = q.shape[0]
+    ang = positions[:T].double()[:, None] * freqs[None, :Dr // 2]
+    cs = (ang.cos().float() * mag)[:, None]
+    sn = (ang.sin().float() * mag)[:, None]
+
+    def turn(x):  # [T, heads, Dr]
+        u, v = x[..., 0::2].float(), x[..., 1::2].float()
+        return torch.stack([u * cs - v * sn, v * cs + u * sn],
+                           -1).flatten(-2)
+
+    heads = q.view(T, H, D + Dr)
+    heads[..., D:] = turn(heads[..., D:]).to(q.dtype)
+    rows = cache.view(-1, R + Dr)
+    slots = slot_mapping[:T]
+    c = ckv[:, :R].float()
+    c = c * torch.rsqrt((c * c).mean(-1, keepdim=True) + eps) * w.float()
+    rows[slots] = torch.cat([c, turn(ckv[:, None, R:])[:, 0]],
+                            -1).to(cache.dtype)
+
+
+def head_gate(x, gate=None):
+    """[H, T, D] -> [T, H*D], times sigmoid(gate)."""
+    H, T, D = x.shape
+    o = x.transpose(0, 1).reshape(T, H * D)
+    if gate is None:
+        return o.contiguous()
+    return (o.float() * torch.sigmoid(gate.float())).to(x.dtype)
 
 
 def hyper_streams(xs, y=None, y2=None, gate=None, mix=None, out_w=None,
@@ -634,6 +681,17 @@ def xielu(x: torch.Tensor, a_pos: float, a_neg: float) -> torch.Tensor:
 def relu2(x: torch.Tensor) -> torch.Tensor:
     r = torch.relu(x.float())
     return (r * r).to(x.dtype)
+
+
+def gelu_erf(x: torch.Tensor) -> torch.Tensor:
+    return torch.nn.functional.gelu(x.float()).to(x.dtype)
+
+
+def token_gate(z, table, ids, col0):
+    """gelu_tanh(z) * the ids' rows of a column block of ``table``."""
+    e = table[ids, col0:col0 + z.shape[1]].float()
+    g = torch.nn.functional.gelu(z.float(), approximate="tanh")
+    return (g * e).to(z.dtype)
 
 
 def topk_then_softmax(logits: torch.Tensor, topk: int):

@@ -44,6 +44,7 @@ class ModelRunner:
                                   else "cuda:0")
         self.model, self.hf_config = load_model(cfg, cfg.device)
         self.kv_dtype = cfg.torch_dtype()
+        cfg.cap_model_length(getattr(self.model, "max_positions", 0))
         if getattr(self.model, "ssm_spec", None) is not None:
             # prefix caching stays ON: page-boundary recurrent-state
             # snapshots restore on hits (core/ssm.py + the hit_filter
