@@ -968,8 +968,19 @@ def latent_attention(q_lat, q_rot, cache, block_table, seq_lens,
     i sees 0 <= i - j < window (window <= 0: every j <= i), ``sinks``
     (fp32 [H]) join the softmax denominator, and the result per head is
     the weighted latent. q_lat [H, T, R], q_rot [T, H, Dr] (views are
-    fine); returns [H, T, R]."""
+    fine); returns [H, T, R].
+
+    bf16 with R <= 512, R + Dr <= 576 and 8-aligned sizes runs the MFMA
+    kernel (prompt portions, mixed batches and, with the keys split,
+    decoding); fp32 and other sizes the generic windowed kernel."""
     H, T, R = q_lat.shape
+    if q_lat.is_cuda and q_lat.dtype == torch.bfloat16:
+        out = torch.empty(H, T, R, dtype=q_lat.dtype, device=q_lat.device)
+        if _seq_kernels().latent_attention_mfma(
+                out, q_lat, q_rot, cache, block_table, seq_lens,
+                query_start_loc, float(scale), int(window), sinks,
+                int(max_query_len)):
+            return out
     v_cache = cache[..., :R]
     q = torch.cat([q_lat.transpose(0, 1), q_rot], -1).reshape(T, -1)
     o = window_attention(q, None, cache, v_cache, block_table, seq_lens,

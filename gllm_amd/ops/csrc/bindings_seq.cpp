@@ -123,6 +123,12 @@ void latent_rope_store(torch::Tensor q, torch::Tensor ckv, torch::Tensor w,
                        torch::Tensor slot_mapping, torch::Tensor freqs,
                        double mag, torch::Tensor cache, long H, long D,
                        long R, long Dr);
+bool latent_attention_mfma(torch::Tensor out, torch::Tensor q_lat,
+                           torch::Tensor q_rot, torch::Tensor cache,
+                           torch::Tensor block_table, torch::Tensor seq_lens,
+                           torch::Tensor query_start_loc, double scale,
+                           long window, c10::optional<torch::Tensor> sinks,
+                           long max_query_len);
 void channel_delta_rule(torch::Tensor o, torch::Tensor q, torch::Tensor k,
                         torch::Tensor v, torch::Tensor a, torch::Tensor b,
                         torch::Tensor A_log, torch::Tensor dt_bias,
@@ -205,6 +211,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("latent_rope_store", &latent_rope_store,
         "latent norm + rotated key part into the paged cache, query heads' "
         "rotated parts in place");
+  m.def("latent_attention_mfma", &latent_attention_mfma,
+        "MFMA attention over a paged latent + rotated key part (bf16); "
+        "false = geometry not instantiated");
   m.def("channel_delta_rule", &channel_delta_rule,
         "ragged gated delta rule with a decay per key channel");
   m.def("gated_act_mul", &gated_act_mul, "act(x[:d]) * x[d:], silu or gelu");

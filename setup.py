@@ -7,12 +7,11 @@ repo snapshots without a site-packages install:
 
 * ``gllm_amd._kernels``      the kernel families of the other models
 * ``gllm_amd._kernels_seq``  the dtype-generic sequence-mixer kernels
-  (layer norm over an fp32 residual, windowed sink attention,
-  talking-heads attention, varlen gated delta rule) plus the grouped
-  MoE GEMM, activations and skinny GEMM that the linear / MoE layers
-  dispatch to — the only native code a Sudevik- or Gukirax-style model
-  needs, so a fresh checkout can serve one after compiling nine files
-  instead of sixteen.
+  (norms over an fp32 residual, windowed sink attention, talking-heads
+  and latent attention, varlen delta rules) plus the grouped MoE GEMM,
+  activations and skinny GEMM that the linear / MoE layers dispatch to —
+  the only native code the config-driven decoder families need, so a
+  fresh checkout can serve one without compiling the rest.
 
 ``GLLM_EXT=seq`` (or ``core``) restricts the build to one module.
 """
@@ -34,7 +33,7 @@ CXX_FLAGS = ["-O3", "-std=c++17"]
 
 SEQ_SOURCES = ["bindings_seq.cpp", "layernorm.hip", "hyper.hip",
                "mingru.hip", "attention_window.hip",
-               "attention_talking.hip",
+               "attention_talking.hip", "attention_latent.hip",
                "attention_prefill.hip", "attention_decode.hip",
                "delta_rule.hip", "moe.hip", "elementwise.hip",
                "skinny_gemm.hip"]
