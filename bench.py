@@ -337,6 +337,36 @@ def sofunex_config(sz, vocab=32000, window=4096):
             "vocab_size": vocab, "width": sz["width"]}
 
 
+def kaketar_config(sz, vocab=32000, window=4096):
+    """Channel-decayed delta layers at the delta geometry of the size
+    table with every fourth layer a latent-attention layer (rotated part
+    and latent of a usual size: half a head, four heads); a dense
+    feed-forward with as many active weights as the table's experts, a
+    side input an eighth of the width wide."""
+    H, _, D = sz["attn"]
+    dh, dg, dk, dv = sz["delta"]
+    mlp = {"kind": "dense", "ff": sz["top"] * sz["ff"] * 3 // 2}
+    layers = []
+    for i in range(sz["layers"]):
+        if (i + 1) % 4 == 0:
+            layers.append({"type": "latent_attention", "mlp": mlp, "mixer": {
+                "heads": H, "dim": D, "rot_dim": D // 2, "vdim": D,
+                "q_rank": sz["width"] * 3 // 4, "kv_rank": 4 * D,
+                "scale": (D + D // 2) ** -0.5, "mask": {"size": window},
+                "rot": {"dims": D // 2, "base": 1000000.0,
+                        "scaling": {"factor": 8.0, "original": 4096,
+                                    "fast": 32.0, "slow": 1.0}}}})
+        else:
+            layers.append({"type": "channel_delta", "mlp": mlp, "mixer": {
+                "heads": dh, "kv_heads": dg, "dim": dk, "vdim": dv,
+                "conv": 4}})
+    return {"architecture": "Kaketar", "embedding": {"scale": 1.0},
+            "layers": layers, "logit_softcap": 30.0,
+            "max_positions": 8192, "norm": {"eps": 1e-5},
+            "token_side": {"dim": sz["width"] // 8}, "vocab": vocab,
+            "vocab_size": vocab, "width": sz["width"]}
+
+
 COMPARE_PAIRS = {
     "sudevik": (("sudevik", sudevik_config),
                 ("hybrid-gdn", hybrid_gdn_config)),
@@ -353,6 +383,12 @@ COMPARE_PAIRS = {
     "sofunex": (("sofunex", sofunex_config),
                 ("gopetar", gopetar_config),
                 ("sudevik", sudevik_config)),
+    # closest existing families: Sudevik (delta rule over the state pool
+    # with every fourth layer attention, norms over an fp32 stream) and
+    # Gopetar (attention over a cached latent)
+    "kaketar": (("kaketar", kaketar_config),
+                ("sudevik", sudevik_config),
+                ("gopetar", gopetar_config)),
 }
 
 
@@ -368,6 +404,8 @@ MODELS["gopetar-w2048"] = ("Gopetar-w2048-8L",
                            gopetar_config(COMPARE_SIZES["w2048"]))
 MODELS["sofunex-w2048"] = ("Sofunex-w2048-8runs",
                            sofunex_config(COMPARE_SIZES["w2048"]))
+MODELS["kaketar-w2048"] = ("Kaketar-w2048-8L",
+                           kaketar_config(COMPARE_SIZES["w2048"]))
 MODELS["sudevik-attn-w2048"] = (
     "Sudevik-attn-w2048-8L",
     sudevik_attention_config(COMPARE_SIZES["w2048"]))

@@ -405,29 +405,39 @@ __global__ __launch_bounds__(LA_BLOCK, 2) void latent_attention_kernel(
 }
 
 // one workgroup per (token, head): weights exp(lse) of the splits, the
-// sink joining the denominator. grid (T * H), block 128.
+// sink joining the denominator. grid (T * H), block 128; splits <= 32.
 __global__ __launch_bounds__(128) void latent_merge_kernel(LatentArgs a) {
+  __shared__ float wt[32];
   const long row = blockIdx.x;
   const int h = row % a.H;
   const long t = row / a.H;
-  const float sink = a.sinks ? a.sinks[h] : -INFINITY;
-  float mx = sink;
-  for (int s = 0; s < a.splits; ++s)
-    mx = fmaxf(mx, a.part_lse[(long)s * a.rows_total + row]);
-  float den = a.sinks ? __expf(sink - mx) : 0.f;
-  for (int s = 0; s < a.splits; ++s)
-    den += __expf(a.part_lse[(long)s * a.rows_total + row] - mx);
-  const float inv = 1.f / den;
+  if (threadIdx.x < WAVE_SIZE) {
+    const int s = threadIdx.x;
+    const float lse =
+        s < a.splits ? a.part_lse[(long)s * a.rows_total + row] : -INFINITY;
+    const float sink = a.sinks ? a.sinks[h] : -INFINITY;
+    const float mx = fmaxf(wave_reduce_max(lse), sink);
+    const float w = __expf(lse - mx);  // 0: that split wrote nothing
+    const float den = wave_reduce_sum(w) + __expf(sink - mx);
+    if (s < 32) wt[s] = w / den;
+  }
+  __syncthreads();
   __hip_bfloat16 *dst = a.out + h * a.out_hs + t * a.out_ts;
-  for (int d = threadIdx.x; d < a.R; d += 128) {
-    float o = 0.f;
+  const float *src = a.part_o + row * a.R;
+  const long step = a.rows_total * a.R;
+  for (int d = threadIdx.x * 4; d < a.R; d += 512) {
+    acc4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
     for (int s = 0; s < a.splits; ++s) {
-      const float lse = a.part_lse[(long)s * a.rows_total + row];
-      if (lse == -INFINITY) continue;  // that split wrote nothing
-      o += __expf(lse - mx) *
-           a.part_o[((long)s * a.rows_total + row) * a.R + d];
+      const float w = wt[s];
+      if (w > 0.f) {
+        const acc4 v = *reinterpret_cast<const acc4 *>(src + s * step + d);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] += w * v[e];
+      }
     }
-    dst[d] = __float2bfloat16(o * inv);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) dst[d + e] = __float2bfloat16(o[e]);
   }
 }
 

@@ -883,6 +883,16 @@ DEV_INLINE float softplus_f(float z) {
   return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
 }
 
+// exp(-rate * softplus(z)): library functions in fp32 serving; with 16-bit
+// logits the hardware exponential and logarithm, log(1 + e) as its series
+// where 1 + e would drop e's bits
+template <typename T> DEV_INLINE float decay_f(float z, float rate) {
+  if (sizeof(T) == 4) return expf(-rate * softplus_f(z));
+  const float e = __expf(-fabsf(z));
+  const float l = e < 1e-3f ? e * (1.0f - 0.5f * e) : __logf(1.0f + e);
+  return __expf(-rate * (fmaxf(z, 0.f) + l));
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void channel_delta_prep_kernel(
     float *__restrict__ scal, float *__restrict__ gdec,
@@ -899,8 +909,8 @@ __global__ __launch_bounds__(256) void channel_delta_prep_kernel(
   const T *ar = a + t * a_stride + (long)h * Dk;
   float *gr = gdec + (t * H + h) * Dk;
   for (int i = lane; i < Dk; i += 64)
-    gr[i] = expf(-rate * softplus_f(ScalarOps<T>::to_f32(ar[i]) +
-                                    dt_bias[(long)h * Dk + i]));
+    gr[i] = decay_f<T>(
+        ScalarOps<T>::to_f32(ar[i]) + dt_bias[(long)h * Dk + i], rate);
   if (lane == 0)
     sc[2 * G + h] =
         1.0f / (1.0f + expf(-ScalarOps<T>::to_f32(bproj[t * b_stride + h])));
@@ -917,6 +927,51 @@ __global__ __launch_bounds__(256) void channel_delta_prep_kernel(
   sk = wave_reduce_sum(sk);
   sq = wave_reduce_sum(sq);
   if (lane == 0) {
+    sc[g] = 1.0f / sqrtf(sk + 1e-6f);
+    sc[G + g] = q_scale / sqrtf(sq + 1e-6f);
+  }
+}
+
+// The same with 16 B accesses: LPH = Dk / 8 lanes per value head, 8
+// channels each. grid (tokens, ceil(H * LPH / 256)), block 256.
+template <typename T, int LPH>
+__global__ __launch_bounds__(256) void channel_delta_prep8_kernel(
+    float *__restrict__ scal, float *__restrict__ gdec,
+    const T *__restrict__ q, const T *__restrict__ k, long qkv_stride,
+    const T *__restrict__ a, long a_stride, const T *__restrict__ bproj,
+    long b_stride, const float *__restrict__ A_log,
+    const float *__restrict__ dt_bias, int H, int G, float q_scale) {
+  constexpr int Dk = LPH * 8;
+  const long t = blockIdx.x;
+  const int h = (blockIdx.y * 256 + threadIdx.x) / LPH;
+  const int d0 = (threadIdx.x % LPH) * 8;
+  if (h >= H) return;  // whole lane groups; no barrier in this kernel
+  float *sc = scal + t * (2 * G + H);
+  const float rate = expf(A_log[h]);
+  float z[8], dt[8];
+  ld8<T>(a + t * a_stride + (long)h * Dk + d0, z);
+  ld8<float>(dt_bias + (long)h * Dk + d0, dt);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) z[e] = decay_f<T>(z[e] + dt[e], rate);
+  st8<float>(gdec + (t * H + h) * Dk + d0, z);
+  if (d0 == 0)
+    sc[2 * G + h] =
+        1.0f / (1.0f + expf(-ScalarOps<T>::to_f32(bproj[t * b_stride + h])));
+  const int per = H / G;
+  if (h % per) return;
+  const int g = h / per;
+  float kf[8], qf[8];
+  ld8<T>(k + t * qkv_stride + (long)g * Dk + d0, kf);
+  ld8<T>(q + t * qkv_stride + (long)g * Dk + d0, qf);
+  float sk = 0.f, sq = 0.f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    sk += kf[e] * kf[e];
+    sq += qf[e] * qf[e];
+  }
+  sk = group_reduce_sum<LPH>(sk);
+  sq = group_reduce_sum<LPH>(sq);
+  if (d0 == 0) {
     sc[g] = 1.0f / sqrtf(sk + 1e-6f);
     sc[G + g] = q_scale / sqrtf(sq + 1e-6f);
   }
@@ -1141,10 +1196,10 @@ __global__ __launch_bounds__(256) void channel_delta_decode_kernel(
     if (tid < Dk) {
       kv = ScalarOps<T>::to_f32(k[t * qkv_stride + (long)g * Dk + tid]);
       qv = ScalarOps<T>::to_f32(q[t * qkv_stride + (long)g * Dk + tid]);
-      gv = expf(-expf(A_log[h]) *
-                softplus_f(ScalarOps<T>::to_f32(
-                               a[t * a_stride + (long)h * Dk + tid]) +
-                           dt_bias[(long)h * Dk + tid]));
+      gv = decay_f<T>(ScalarOps<T>::to_f32(
+                          a[t * a_stride + (long)h * Dk + tid]) +
+                          dt_bias[(long)h * Dk + tid],
+                      expf(A_log[h]));
     }
     ks[tid] = kv;
     qs[tid] = qv;
@@ -1700,8 +1755,32 @@ void channel_delta_rule(torch::Tensor o, torch::Tensor q, torch::Tensor k,
                      (const TT *)b.data_ptr(), (long)b.stride(0),            \
                      A_log.data_ptr<float>(), dt_bias.data_ptr<float>(), H,  \
                      G, Dk, (float)q_scale)
-  if (st == at::kBFloat16) PREP(__hip_bfloat16);
-  else PREP(float);
+#define PREP8(TT, L)                                                         \
+  hipLaunchKernelGGL((channel_delta_prep8_kernel<TT, L>),                    \
+                     dim3(T, (H * L + 255) / 256), dim3(256), 0, stream,     \
+                     scal.data_ptr<float>(), gdec.data_ptr<float>(),         \
+                     (const TT *)q.data_ptr(), (const TT *)k.data_ptr(),     \
+                     (long)q.stride(0), (const TT *)a.data_ptr(),            \
+                     (long)a.stride(0), (const TT *)b.data_ptr(),            \
+                     (long)b.stride(0), A_log.data_ptr<float>(),             \
+                     dt_bias.data_ptr<float>(), H, G, (float)q_scale)
+#define PREP_L(TT)                                                           \
+  if (!vec8) PREP(TT);                                                       \
+  else if (Dk == 32) PREP8(TT, 4);                                           \
+  else if (Dk == 64) PREP8(TT, 8);                                           \
+  else if (Dk == 128) PREP8(TT, 16);                                         \
+  else PREP8(TT, 32)
+  const size_t es = q.element_size();
+  auto al16 = [&](const torch::Tensor &x) {
+    return reinterpret_cast<uintptr_t>(x.data_ptr()) % 16 == 0 &&
+           (x.dim() < 2 || (x.stride(0) * es) % 16 == 0);
+  };
+  const bool vec8 = (Dk == 32 || Dk == 64 || Dk == 128 || Dk == 256) &&
+                    al16(q) && al16(k) && al16(a) && al16(dt_bias);
+  if (st == at::kBFloat16) { PREP_L(__hip_bfloat16); }
+  else { PREP_L(float); }
+#undef PREP_L
+#undef PREP8
 #undef PREP
   // a few sequences leave most of the chip idle at 64 columns a workgroup:
   // sixteen lanes per column then shorten every token's chain
