@@ -981,12 +981,15 @@ def latent_attention(q_lat, q_rot, cache, block_table, seq_lens,
                 query_start_loc, float(scale), int(window), sinks,
                 int(max_query_len)):
             return out
-    v_cache = cache[..., :R]
     q = torch.cat([q_lat.transpose(0, 1), q_rot], -1).reshape(T, -1)
-    o = window_attention(q, None, cache, v_cache, block_table, seq_lens,
-                         query_start_loc, scale, window, 0, False,
-                         max_query_len, sinks=sinks)
-    return o.view(T, H, R).transpose(0, 1)
+    # (the generic kernel holds up to 512 value columns)
+    parts = [window_attention(q, None, cache, cache[..., c:min(c + 512, R)],
+                              block_table, seq_lens, query_start_loc, scale,
+                              window, 0, False, max_query_len,
+                              sinks=sinks).view(T, H, -1)
+             for c in range(0, R, 512)]
+    o = parts[0] if len(parts) == 1 else torch.cat(parts, -1)
+    return o.transpose(0, 1)
 
 
 def head_gate(x, gate=None) -> torch.Tensor:
